@@ -504,7 +504,7 @@ LS_DEFINE_ERROR_API
 // The entry points that a list of launches may name (the kernels of a layer).
 #define LS_CORE_LISTED(X)                                                                                        \
   X(ls_gemm) X(ls_gemm_slices) X(ls_gemm_slices_folded) X(ls_add_rmsnorm) X(ls_rmsnorm) X(ls_qk_rope_kv) X(ls_swiglu) \
-  X(ls_bias_act) X(ls_embed)
+  X(ls_bias_act) X(ls_embed) X(ls_gemm_xielu)
 LS_DEFINE_LISTED_CALLS(LS_CORE_LISTED)
 
 extern "C" int ls_run_list(const long long* words, long n_words, long* failed_at) {

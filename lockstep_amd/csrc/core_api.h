@@ -69,6 +69,8 @@ int ls_advance_decode(int* meta, long meta_ints, int n_seqs, int off_tokens, con
 // Matrix products C = X W^T with a fixed summation order (see gemm.hip).
 int ls_gemm(int dtype, int epilogue, const void* X, const void* W, void* C, int M, int N, int K, long ldx, long ldc,
             const float* norm_w, float eps, int out_cols, void* stream);
+int ls_gemm_xielu(int dtype, const void* X, const void* W, void* C, int M, int N, int K, long ldx, long ldc,
+                  const float* act, void* stream);
 int ls_gemm_kslice(int K);
 int ls_gemm_slices_count(int K);
 int ls_gemm_slices_max_rows(int dtype, int K);

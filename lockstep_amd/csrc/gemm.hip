@@ -83,6 +83,7 @@ enum Epilogue : int {
                   // C[m][16t + i] = (g * 1/(1 + exp(-g))) * u in float, stored in the compute dtype
   kSliceSums = 4, // the tiled kernel only: C is float [slices][M][N] and gets the sums of the K slices, not their
                   // total; the workgroups with blockIdx.y = y take the slices [y * out_cols, (y + 1) * out_cols)
+  kXielu = 5,     // C[m][n] = xielu(total) in the compute dtype, the activation's two factors from act[0], act[1]
 };
 
 __host__ __device__ inline int kslice_for(int K) { return 256 * ((K + 4095) / 4096); }
@@ -141,6 +142,23 @@ __device__ __forceinline__ void epilogue_swiglu4(void* __restrict__ C, long ldc,
   epilogue4<T, kStore>(C, ldc, m, col, M, width, act, vec_ok);
 }
 
+// xIELU of a float total:  up z^2 + z/2 above zero,  down (e^z - 1 - z) + z/2 elsewhere.
+__device__ __forceinline__ float xielu(float z, float up, float down) {
+  const float low = fminf(z, 0.f);
+  return (z > 0.f ? up * (z * z) : down * (expm1f(low) - low)) + 0.5f * z;
+}
+
+template <typename T>
+__device__ __forceinline__ void epilogue_xielu4(void* __restrict__ C, long ldc, int m, int n, int M, int N,
+                                                const float total[4], bool vec_ok, const float* __restrict__ act) {
+  if (m >= M || n >= N) return;
+  const float up = act[0], down = act[1];
+  float v[4];
+#pragma unroll
+  for (int r = 0; r < 4; ++r) v[r] = xielu(total[r], up, down);
+  epilogue4<T, kStore>(C, ldc, m, n, M, N, v, vec_ok);
+}
+
 // RMSNorm of rows of the float residual stream, as a prologue of the skinny
 // kernel (at most 16 rows): the sum of squares of a row is formed exactly as
 // rmsnorm_kernel forms it (row_sumsq_part over the first 256 threads, a
@@ -185,7 +203,7 @@ __global__ __launch_bounds__(NW * 64) void gemm_skinny_kernel(const void* __rest
                                                                void* __restrict__ C, int M, int N, int K, long ldx,
                                                                long ldc, int kslice, int aligned, int vec_ok,
                                                                const float* __restrict__ norm_w, float eps,
-                                                               int out_cols) {
+                                                               int out_cols, const float* __restrict__ act) {
   typedef Atom<T> A;
   typedef typename A::vec_t vec_t;
   constexpr int NT = (EPI == kSwiGLU) ? 2 : 1;  // weight tiles per workgroup
@@ -319,6 +337,8 @@ __global__ __launch_bounds__(NW * 64) void gemm_skinny_kernel(const void* __rest
     const int m = j * 16 + (l & 15);
     if (EPI == kSwiGLU)
       epilogue_swiglu4<T>(C, ldc, m, blockIdx.x * 16 + (l >> 4) * 4, M, out_cols, total[0], total[NT - 1], vec_ok);
+    else if constexpr (EPI == kXielu)
+      epilogue_xielu4<T>(C, ldc, m, n0 + (l >> 4) * 4, M, N, total[0], vec_ok, act);
     else
       epilogue4<T, EPI>(C, ldc, m, n0 + (l >> 4) * 4, M, N, total[0], vec_ok,
                         (preload && idx == (int)threadIdx.x) ? &old_vals : nullptr);
@@ -341,7 +361,8 @@ template <typename T, int MT, int EPI, int XC>
 __global__ __launch_bounds__(1024) void gemm_stream_kernel(const T* __restrict__ X, const T* __restrict__ W,
                                                            void* __restrict__ C, int M, int N, int K, long ldx,
                                                            long ldc, int kslice, int aligned, int vec_ok,
-                                                           int out_cols, int blocks, int row_groups) {
+                                                           int out_cols, int blocks, int row_groups,
+                                                           const float* __restrict__ act) {
   typedef Atom<T> A;
   typedef typename A::vec_t vec_t;
   constexpr int NT = (EPI == kSwiGLU) ? 2 : 1;  // weight tiles per column block
@@ -451,6 +472,8 @@ __global__ __launch_bounds__(1024) void gemm_stream_kernel(const T* __restrict__
       const int m = m_base + j * 16 + row16;
       if (EPI == kSwiGLU)
         epilogue_swiglu4<T>(C, ldc, m, b * 16 + g * 4, M, out_cols, total[0], total[NT - 1], vec_ok);
+      else if constexpr (EPI == kXielu)
+        epilogue_xielu4<T>(C, ldc, m, b * 16 + g * 4, M, N, total[0], vec_ok, act);
       else
         epilogue4<T, EPI>(C, ldc, m, b * 16 + g * 4, M, N, total[0], vec_ok);
     }
@@ -867,7 +890,7 @@ template <typename T, int EPI, int BM, int BN, int PD, bool AL, int NWM = 2, int
 __global__ __launch_bounds__(64 * NWM * NWN) void gemm_tiled_kernel(const T* __restrict__ X, const T* __restrict__ W,
                                                          void* __restrict__ C, int M, int N, int K, long ldx,
                                                          long ldc, int kslice, int vec_ok, int tiles_m, int tiles_n,
-                                                         int out_cols) {
+                                                         int out_cols, const float* __restrict__ act) {
   typedef Atom<T> A;
   typedef typename A::vec_t vec_t;
   constexpr int BK = kRowBytes / sizeof(T);  // elements of K per stage
@@ -1075,14 +1098,17 @@ __global__ __launch_bounds__(64 * NWM * NWN) void gemm_tiled_kernel(const T* __r
 #pragma unroll
       for (int j = 0; j < TJ; ++j) {
         float t[4] = {total[i][j][0], total[i][j][1], total[i][j][2], total[i][j][3]};
-        epilogue4<T, EPI>(C, ldc, m_base + wm + j * 16 + row16, n_base + wn + i * 16 + g * 4, M, N, t, vec_ok);
+        if constexpr (EPI == kXielu)
+          epilogue_xielu4<T>(C, ldc, m_base + wm + j * 16 + row16, n_base + wn + i * 16 + g * 4, M, N, t, vec_ok, act);
+        else
+          epilogue4<T, EPI>(C, ldc, m_base + wm + j * 16 + row16, n_base + wn + i * 16 + g * 4, M, N, t, vec_ok);
       }
   }
 }
 
 template <typename T, int EPI>
 int launch_gemm(const void* X, const void* W, void* C, int M, int N, int K, long ldx, long ldc, const float* norm_w,
-                float eps, int out_cols, hipStream_t stream) {
+                float eps, int out_cols, hipStream_t stream, const float* act = nullptr) {
   int kslice = kslice_for(K);
   if (LS_MUTANT_HOST(kMutantKsliceByRows) && M > 16 && M <= 64) kslice *= 2;  // the mutant: K blocking that depends on the rows of the launch
   const int nslices = (K + kslice - 1) / kslice;
@@ -1090,7 +1116,7 @@ int launch_gemm(const void* X, const void* W, void* C, int M, int N, int K, long
   constexpr int NT = (EPI == kSwiGLU) ? 2 : 1;
   const int aligned = (K % VEC == 0) && (norm_w || ldx % VEC == 0) && (reinterpret_cast<uintptr_t>(X) % 16 == 0) &&
                       (reinterpret_cast<uintptr_t>(W) % 16 == 0);
-  const size_t out_size = (EPI == kStore || EPI == kSwiGLU) ? sizeof(T) : sizeof(float);
+  const size_t out_size = (EPI == kStore || EPI == kSwiGLU || EPI == kXielu) ? sizeof(T) : sizeof(float);
   const int vec_ok = (ldc % 4 == 0) && (reinterpret_cast<uintptr_t>(C) % (4 * out_size) == 0);
   const T* w = reinterpret_cast<const T*>(W);
   if (norm_w && M > 16) return fail("gemm: the fused norm prologue takes at most 16 rows, got %d", M);
@@ -1129,7 +1155,7 @@ int launch_gemm(const void* X, const void* W, void* C, int M, int N, int K, long
   if (stream_lds_ready<T, MT_, EPI, XC_>(stream_lds))                                                             \
     hipLaunchKernelGGL((gemm_stream_kernel<T, MT_, EPI, XC_>), grid, dim3(nslices * 64), stream_lds, stream,      \
                        reinterpret_cast<const T*>(X), w, C, M, N, K, ldx, ldc, kslice, aligned, vec_ok, out_cols, \
-                       col_blocks, row_groups);                                                                   \
+                       col_blocks, row_groups, act);                                                              \
   else                                                                                                            \
     launched = false
     if (group_tiles == 1 && xc == 8) LS_STREAM(1, 8);
@@ -1149,7 +1175,7 @@ int launch_gemm(const void* X, const void* W, void* C, int M, int N, int K, long
       const int tiles_n = (N + 31) / 32;
       hipLaunchKernelGGL((gemm_tiled_kernel<T, EPI, 64, 32, LS_GEMM_PD_SMALL, true, 2, 2>), dim3(tiles_n), dim3(256), 0,
                          stream, reinterpret_cast<const T*>(X), w, C, M, N, K, ldx, ldc, kslice, vec_ok, 1, tiles_n,
-                         out_cols);
+                         out_cols, act);
       return check_launch("gemm");
     }
   }
@@ -1161,9 +1187,11 @@ int launch_gemm(const void* X, const void* W, void* C, int M, int N, int K, long
     const size_t lds = ((size_t)nslices * NT * mt * 256 + (norm_w ? 80 : 0)) * sizeof(float);
 #define LS_SKINNY(MT_, NW_, NORM_)                                                                              \
   hipLaunchKernelGGL((gemm_skinny_kernel<T, MT_, NW_, EPI, NORM_>), grid, dim3(NW_ * 64), lds, stream, X, w, C, M, N, \
-                     K, ldx, ldc, kslice, aligned, vec_ok, norm_w, eps, out_cols)
+                     K, ldx, ldc, kslice, aligned, vec_ok, norm_w, eps, out_cols, act)
     if (norm_w) {
-      if (nw >= 8) LS_SKINNY(1, 8, true); else LS_SKINNY(1, 4, true);
+      if constexpr (EPI == kXielu) return fail("gemm: the xIELU epilogue has no norm prologue");
+      else if (nw >= 8) LS_SKINNY(1, 8, true);
+      else LS_SKINNY(1, 4, true);
     } else if (nw == 16) {
       if (mt == 1) LS_SKINNY(1, 16, false); else LS_SKINNY(2, 16, false);
     } else if (nw == 8) {
@@ -1183,7 +1211,7 @@ int launch_gemm(const void* X, const void* W, void* C, int M, int N, int K, long
     const int tiles_m = (M + BM_ - 1) / BM_, tiles_n = (N + BN_ - 1) / BN_;                                       \
     hipLaunchKernelGGL((gemm_tiled_kernel<T, EPI, BM_, BN_, PD_, AL_, NWM_, NWN_>), dim3(tiles_m * tiles_n),      \
                        dim3(64 * NWM_ * NWN_), 0, stream, reinterpret_cast<const T*>(X), w, C, M, N, K, ldx, ldc, \
-                       kslice, vec_ok, tiles_m, tiles_n, out_cols);                                             \
+                       kslice, vec_ok, tiles_m, tiles_n, out_cols, act);                                        \
   }
 #define LS_TILED(BM_, BN_, PD_, AL_) LS_TILED_WAVES(BM_, BN_, PD_, AL_, 2, 2)
     // 128 x 256 tiles load a quarter fewer operand bytes per MFMA (measured at 2,048 rows: gate and up of
@@ -1244,6 +1272,20 @@ extern "C" int ls_gemm(int dtype, int epilogue, const void* X, const void* W, vo
   if (dtype == kBF16) { LS_GEMM_CASE(bf16_t) }
 #undef LS_GEMM_CASE
   return fail("gemm: unknown dtype %d", dtype);
+}
+
+// C [M][N] (dtype) = xielu(X @ W^T), elementwise: act[0] z^2 + z/2 for z > 0, act[1] (e^z - 1 - z) + z/2 elsewhere;
+// act: two floats on the device.  Operands as for ls_gemm.
+extern "C" int ls_gemm_xielu(int dtype, const void* X, const void* W, void* C, int M, int N, int K, long ldx, long ldc,
+                             const float* act, void* stream) {
+  using namespace ls;
+  LS_REQUIRE(M > 0 && N > 0 && K > 0, "gemm_xielu: sizes must be positive, got M=%d N=%d K=%d", M, N, K);
+  LS_REQUIRE(ldx >= K && ldc >= N, "gemm_xielu: row strides ldx=%ld ldc=%ld are shorter than K=%d / N=%d", ldx, ldc, K, N);
+  LS_REQUIRE(X && W && C && act, "gemm_xielu: null operand");
+  hipStream_t s = reinterpret_cast<hipStream_t>(stream);
+  if (dtype == kF32) return launch_gemm<float, kXielu>(X, W, C, M, N, K, ldx, ldc, nullptr, 0.f, N, s, act);
+  if (dtype == kBF16) return launch_gemm<bf16_t, kXielu>(X, W, C, M, N, K, ldx, ldc, nullptr, 0.f, N, s, act);
+  return fail("gemm_xielu: unknown dtype %d", dtype);
 }
 
 extern "C" int ls_gemm_kslice(int K) { return ls::kslice_for(K); }
@@ -1318,7 +1360,7 @@ extern "C" int ls_gemm_slices(int dtype, const void* X, const void* W, float* P,
       dim3 tiled_grid(tiles_m * tiles_n, groups_y);
 #define LS_TILED_SLICES(T_)                                                                                          \
   hipLaunchKernelGGL((gemm_tiled_kernel<T_, kSliceSums, 64, 64, LS_GEMM_PD_SMALL, true, 2, 2>), tiled_grid, dim3(256), \
-                     0, s, (const T_*)X, (const T_*)W, (void*)P, M, N, K, ldx, (long)N, kslice, 1, tiles_m, tiles_n, per)
+                     0, s, (const T_*)X, (const T_*)W, (void*)P, M, N, K, ldx, (long)N, kslice, 1, tiles_m, tiles_n, per, (const float*)nullptr)
       if (dtype == kF32) { LS_TILED_SLICES(float); } else if (dtype == kBF16) { LS_TILED_SLICES(bf16_t); } else return fail("gemm_slices: unknown dtype %d", dtype);
 #undef LS_TILED_SLICES
       return check_launch("gemm_slices");

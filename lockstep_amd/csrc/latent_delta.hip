@@ -146,7 +146,8 @@ __global__ __launch_bounds__(256) void streams_step_kernel(float* __restrict__ X
 // ---------------------------------------------------------------------------
 // Post pass of the down projections of attention over a latent: raw [T][ld] float = a (QR) | c (CR) | r (RD), the
 // last two absent for a layer that reads another layer's latent (has_kv == 0).
-//   a -> a / sqrt(mean(a^2) + eps) * a_weight            -> a_out [T][QR] (T)
+//   a -> a / sqrt(mean(a^2) + eps) * a_weight            -> a_out [T][QR] (T); as it is where a_weight is null (queries
+//                                                           that do not pass a latent)
 //   c -> c / sqrt(mean(c^2) + eps) * c_weight            -> key pages [page][0][slot][0 .. CR) and value pages
 //                                                           [page][0][0 .. CR)[slot]: the latent is key and value
 //   r -> rotated in neighbouring pairs (2i, 2i + 1) on its first `rot` dimensions at the token's position
@@ -163,10 +164,12 @@ __global__ __launch_bounds__(256) void latent_post_kernel(
   __shared__ float scratch[4];
   const int t = blockIdx.x;
   const float* row = raw + (long)t * ld;
-  {
+  if (a_weight) {
     const float part = row_sumsq_part(row, QR, threadIdx.x, false);
     const float scale = 1.0f / sqrtf(block_sum4(part, scratch) / (float)QR + eps);
     for (int e = threadIdx.x; e < QR; e += 256) a_out[(long)t * lda + e] = from_f32<T>((row[e] * scale) * a_weight[e]);
+  } else {
+    for (int e = threadIdx.x; e < QR; e += 256) a_out[(long)t * lda + e] = from_f32<T>(row[e]);
   }
   if (!has_kv) return;
   const int pos = tok_pos[t];
@@ -542,7 +545,7 @@ extern "C" int ls_latent_post(int dtype, const float* raw, long ld, int n_tokens
                               const float* sin_table, int rot, int table_positions, int max_pos, const int* tok_seq,
                               const int* tok_pos, const void* seqs, const int* table, int table_stride, void* a_out,
                               long lda, void* k_pages, void* v_pages, int page_size, void* stream) {
-  LS_REQUIRE(n_tokens > 0 && QR > 0 && raw && a_out && a_weight && lda >= QR && eps > 0.f, "latent_post: bad query latent");
+  LS_REQUIRE(n_tokens > 0 && QR > 0 && raw && a_out && lda >= QR && eps > 0.f, "latent_post: bad query latent");
   LS_REQUIRE(ld >= QR + (has_kv ? CR + RD : 0), "latent_post: rows of %ld floats are too short", ld);
   if (has_kv) {
     LS_REQUIRE(CR > 0 && RD >= 0 && Dp >= CR + RD && c_weight && k_pages && v_pages && table && seqs && tok_seq && tok_pos &&

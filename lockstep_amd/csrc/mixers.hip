@@ -653,7 +653,8 @@ __global__ __launch_bounds__(256) void add_rmsnorm_shift_kernel(float* __restric
 LS_DEFINE_ERROR_API
 
 #define LS_MIXERS_LISTED(X) \
-  X(ls_dyt) X(ls_glu_clamped) X(ls_softcap) X(ls_talk_qkv) X(ls_linrec) X(ls_head_norm_gate)
+  X(ls_dyt) X(ls_glu_clamped) X(ls_softcap) X(ls_talk_qkv) X(ls_linrec) X(ls_head_norm_gate)                  \
+  X(ls_residual_step) X(ls_channel_recurrence)
 LS_DEFINE_LISTED_CALLS(LS_MIXERS_LISTED)
 
 using namespace ls;

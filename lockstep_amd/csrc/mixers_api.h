@@ -116,6 +116,27 @@ int ls_delta_rule(const float* raw, long ld, int n_tokens, int G, int H, int D, 
                   const void* seqs, int n_seqs, float* state, long state_stride, float* scratch, float* out, long ldo,
                   const float* chan, long ldc, void* stream);
 
+// Between two sublayers of a residual stream X [.][width] float (see sublayers.hip): y = P[0][row] + P[1][row] + ...;
+// x = X[row] + norm(y) (post_w null: + y); results[keep][row] = x (results [.][r_rows][width] or null); x = the sum of
+// shares[j] results[j][row] over j = 0 .. keep (shares null: x); X[row] = x; out = norm(x).  A norm subtracts the row's
+// mean when `centred`.  rows: the rows to read, or null for the first n_rows; with it only out is written.
+int ls_residual_step_max_width();
+int ls_residual_step(int dtype, float* X, long ldx, int width, const float* P, int slices, int p_rows, const float* post_w,
+                     float post_eps, int post_centred, float* results, int r_rows, int keep, const float* shares,
+                     const float* weight, float eps, int centred, void* out, long ld_out, const int* rows, int n_rows,
+                     void* stream);
+
+// One number a channel: S_t = (1 - z) S_(t-1) + z c with z = sigmoid(a + a_b), c = v + 1/2 where v = u + u_b >= 0, else
+// sigmoid(v); out = S_t silu(g).  raw [T][ld] float holds a, u and g (width each) at a_at, u_at, g_at; state
+// [slots][state_stride] float.  single_tokens: every request of the step brings one token.
+int ls_channel_recurrence(int dtype, const float* raw, long ld, int a_at, int u_at, int g_at, const float* a_b,
+                          const float* u_b, int width, const void* seqs, int n_seqs, int single_tokens, float* state,
+                          long state_stride, void* out, long ldo, void* stream);
+
+// out [T][ld_out] float = table[token] * scale + (sin(p freq[i]), cos(p freq[i])) at the elements (2i, 2i + 1).
+int ls_embed_positions(int dtype, const int* tokens, const int* tok_pos, const void* table, int vocab, const double* freq,
+                       float* out, int n_tokens, int width, long ld_out, float scale, void* stream);
+
 int ls_listed_index(const char* name);
 int ls_call_listed(int index, const long long* words, int n);
 

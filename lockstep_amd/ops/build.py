@@ -10,7 +10,9 @@ Two kinds of library exist:
 ``mixers``          Dynamic Tanh norm, clamped gated unit, soft cap, the linear
                     recurrence with per-row gates and what surrounds it; the step of
                     a residual stream of several copies, the passes around attention
-                    over a latent, a product a head, the gated delta rule;
+                    over a latent, a product a head, the gated delta rule; the step
+                    between sublayers that are normalised on both sides, with an average
+                    over depth, a recurrence of one number a channel, position vectors;
 ``talking<shape>``  attention whose heads' scores are mixed before the softmax,
                     for one shape (query heads, kv heads, key and value size).
 ``sink<D>x<DV>``    grouped-query attention with a sink in the softmax, windows or
@@ -50,7 +52,7 @@ FLAGS = [
 ]
 CORE_SOURCES = ("core.hip", "gemm.hip", "sample.hip")
 ATTENTION_SOURCES = ("attention.hip",)
-MIXERS_SOURCES = ("mixers.hip", "latent_delta.hip")
+MIXERS_SOURCES = ("mixers.hip", "latent_delta.hip", "sublayers.hip")
 TALKING_SOURCES = ("talking_attention.hip",)
 SINK_SOURCES = ("sink_attention.hip",)
 EXPERTS_SOURCES = ("experts.hip",)

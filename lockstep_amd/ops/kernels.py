@@ -241,6 +241,23 @@ class Kernels:
             c_int(DTYPE_CODE[w.dtype]), c_int(epilogue), _ptr(x), _ptr(w), _ptr(out), c_int(m), c_int(n), c_int(k),
             c_long(x.stride(0)), c_long(out.stride(0)), _ptr(norm_weight), c_float(eps), c_int(cols), _stream()))
 
+    def gemm_xielu(self, x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, act: torch.Tensor) -> None:
+        """``out = xielu(x @ w.T)`` in the compute dtype, element by element: ``act[0] z^2 + z/2`` above zero, ``act[1]
+        (e^z - 1 - z) + z/2`` elsewhere; ``act`` two float32 numbers on the GPU."""
+        _rows_ok(x, "gemm_xielu x"); _rows_ok(w, "gemm_xielu w"); _rows_ok(out, "gemm_xielu out")
+        m, k = x.shape
+        n = w.shape[0]
+        if not (w.dtype in DTYPE_CODE and x.dtype == w.dtype == out.dtype and w.is_contiguous() and w.shape[1] == k
+                and tuple(out.shape) == (m, n)):
+            raise KernelError(f"gemm_xielu: operands {tuple(x.shape)} {x.dtype}, {tuple(w.shape)} {w.dtype} and output "
+                              f"{tuple(out.shape)} {out.dtype} do not fit")
+        self._f32_vector(act, 2, "gemm_xielu act")
+        if m == 0:
+            return
+        self._launch(self.core, self.core.ls_gemm_xielu, (
+            c_int(DTYPE_CODE[w.dtype]), _ptr(x), _ptr(w), _ptr(out), c_int(m), c_int(n), c_int(k), c_long(x.stride(0)),
+            c_long(out.stride(0)), _ptr(act), _stream()))
+
     def gemm_slices_count(self, k: int) -> int:
         """K slices of a product over ``k`` (first dimension of ``gemm_slices``'s output)."""
         return self._memo(("slices", k), lambda: int(self.core.ls_gemm_slices_count(c_int(k))))
@@ -1254,7 +1271,7 @@ class Kernels:
                     has_kv: bool, q_weight, kv_weight, eps: float, cos, sin, rot: int, max_pos: int, tok_seq, tok_pos,
                     seqs, table, q_latent: torch.Tensor, k_pages, v_pages, page_size: int) -> None:
         """Post pass of the down projections ``raw`` (float32, ``a | c | r``): the query latent ``a`` normalised
-        with ``q_weight`` into ``q_latent``; with ``has_kv`` the latent ``c`` normalised with ``kv_weight`` into the
+        with ``q_weight`` (None: as it is) into ``q_latent``; with ``has_kv`` the latent ``c`` normalised with ``kv_weight`` into the
         key pages (dimensions ``0 .. kv_rank`` of the one key head of ``key_pad`` elements) and into the value
         pages, and the shared key part ``r``, rotated in neighbouring pairs on its first ``rot`` dimensions,
         behind it in the key pages."""
@@ -1264,7 +1281,8 @@ class Kernels:
             raise KernelError(f"latent_post raw must be float32 [>= {n_tokens}, >= {width}]")
         if not (q_latent.dtype in DTYPE_CODE and q_latent.shape[0] >= n_tokens and q_latent.shape[1] == q_rank):
             raise KernelError("latent_post q_latent has the wrong shape or dtype")
-        self._f32_vector(q_weight, q_rank, "latent_post q_weight")
+        if q_weight is not None:
+            self._f32_vector(q_weight, q_rank, "latent_post q_weight")
         positions = 0
         if has_kv:
             self._f32_vector(kv_weight, kv_rank, "latent_post kv_weight")
@@ -1476,6 +1494,106 @@ class Kernels:
             c_int(DTYPE_CODE[out.dtype]), _ptr(normed), c_long(normed.stride(0)), _ptr(mu), _ptr(tok_seq), _ptr(tok_pos),
             _ptr(seqs), _ptr(state), c_long(state.stride(0)), _ptr(out), c_long(out.stride(0)), c_int(t), c_int(width),
             _stream()))
+
+    # -- sublayers with norms on both sides, averages over depth ------------------------------------
+    def residual_step(self, x: torch.Tensor, partials, post, results, keep: int, shares, norm, out,
+                      rows: torch.Tensor | None = None) -> None:
+        """One step of the float32 residual stream ``x [T, width]`` between two sublayers.  With ``partials [slices, T,
+        width]`` (a sublayer's output as slice sums, added in ascending order to ``y``): ``x += y``, or, with ``post``,
+        ``x += norm(y)``.  With ``results [layers + 1, T, width]``: ``results[keep] = x``; with ``shares [keep + 1]`` then
+        ``x = sum_j shares[j] results[j]``.  With ``out [rows, width]``: ``out = norm(x)``.  ``post`` and ``norm`` are
+        ``(weight, eps, centred)``; a norm is ``(v - m) / sqrt(mean((v - m)^2) + eps) * weight`` with ``m`` the row's mean
+        if ``centred``, else 0.  ``rows`` selects rows of ``x``; then nothing but ``out`` is written."""
+        _rows_ok(x, "residual_step x")
+        t, width = x.shape
+        lib = self.mixers_lib()
+        widest = self._memo(("residual_step_max",), lambda: int(lib.ls_residual_step_max_width()))
+        if not (x.dtype == torch.float32 and width <= widest):
+            raise KernelError(f"residual_step works on float32 rows of up to {widest} elements")
+        n_rows = t if rows is None else rows.shape[0]
+        if rows is not None and not (rows.is_cuda and rows.dtype == torch.int32 and rows.is_contiguous() and out is not None):
+            raise KernelError("residual_step rows: int32 on the GPU, and an output")
+        slices = p_rows = r_rows = 0
+        if partials is not None:
+            if not (partials.is_cuda and partials.dtype == torch.float32 and partials.is_contiguous() and partials.dim() == 3
+                    and partials.shape[2] == width and partials.shape[1] >= t):
+                raise KernelError(f"residual_step partials must be float32 [slices, >= {t}, {width}]")
+            slices, p_rows = partials.shape[0], partials.shape[1]
+        post_weight, post_eps, post_centred = post if post is not None else (None, 0.0, False)
+        if post is not None:
+            if partials is None:
+                raise KernelError("residual_step: a norm of the sublayer's output needs its slices")
+            self._f32_vector(post_weight, width, "residual_step post weight")
+        if results is not None:
+            if not (results.is_cuda and results.dtype == torch.float32 and results.is_contiguous() and results.dim() == 3
+                    and results.shape[2] == width and results.shape[1] >= t and 0 <= keep < results.shape[0]):
+                raise KernelError(f"residual_step results must be float32 [> {keep}, >= {t}, {width}]")
+            r_rows = results.shape[1]
+        if shares is not None:
+            if results is None:
+                raise KernelError("residual_step: shares need results")
+            self._f32_vector(shares, keep + 1, "residual_step shares")
+        weight, eps, centred, dtype, ld_out = None, 0.0, False, torch.float32, 0
+        if out is not None:
+            weight, eps, centred = norm
+            _rows_ok(out, "residual_step out")
+            if not (out.dtype in DTYPE_CODE and tuple(out.shape) == (n_rows, width) and eps > 0):
+                raise KernelError(f"residual_step out must be [{n_rows},{width}], eps positive")
+            self._f32_vector(weight, width, "residual_step weight")
+            dtype, ld_out = out.dtype, out.stride(0)
+        elif partials is None and results is None:
+            return
+        if n_rows == 0:
+            return
+        self._launch(lib, lib.ls_residual_step, (
+            c_int(DTYPE_CODE[dtype]), _ptr(x), c_long(x.stride(0)), c_int(width), _ptr(partials), c_int(slices), c_int(p_rows),
+            _ptr(post_weight), c_float(post_eps), c_int(int(post_centred)), _ptr(results), c_int(r_rows), c_int(keep),
+            _ptr(shares), _ptr(weight), c_float(eps), c_int(int(centred)), _ptr(out), c_long(ld_out), _ptr(rows), c_int(n_rows),
+            _stream()))
+
+    def channel_recurrence(self, raw: torch.Tensor, a_at: int, u_at: int, g_at: int, a_bias, u_bias, seqs, n_seqs: int,
+                           single_tokens: bool, state: torch.Tensor, out: torch.Tensor) -> None:
+        """``S_t = (1 - z) S_(t-1) + z c``, ``out_t = S_t silu(g)`` element by element over the tokens of every request, with
+        ``z = sigmoid(a + a_bias)`` and ``c = v + 1/2`` where ``v = u + u_bias >= 0``, else ``sigmoid(v)``.  ``raw`` float32
+        rows that hold ``a``, ``u`` and ``g`` at the columns ``a_at``, ``u_at``, ``g_at``; ``state`` float32 ``[slots, width]``."""
+        _rows_ok(raw, "channel_recurrence raw"); _rows_ok(out, "channel_recurrence out")
+        t, width = out.shape
+        if not (raw.dtype == torch.float32 and raw.shape[0] >= t and min(a_at, u_at, g_at) >= 0
+                and raw.shape[1] >= max(a_at, u_at, g_at) + width and out.dtype in DTYPE_CODE):
+            raise KernelError("channel_recurrence: the projections do not fit the float32 rows, or the output's dtype is wrong")
+        self._f32_vector(a_bias, width, "channel_recurrence a_bias"); self._f32_vector(u_bias, width, "channel_recurrence u_bias")
+        if not (state.is_cuda and state.dtype == torch.float32 and state.dim() == 2 and state.stride(1) == 1
+                and state.shape[1] >= width):
+            raise KernelError(f"channel_recurrence state must be float32 [slots, >= {width}]")
+        if not (seqs.is_cuda and seqs.dtype == torch.int32 and seqs.is_contiguous() and seqs.numel() >= 8 * n_seqs):
+            raise KernelError("channel_recurrence seqs: eight int32 a request")
+        if t == 0:
+            return
+        lib = self.mixers_lib()
+        self._launch(lib, lib.ls_channel_recurrence, (
+            c_int(DTYPE_CODE[out.dtype]), _ptr(raw), c_long(raw.stride(0)), c_int(a_at), c_int(u_at), c_int(g_at),
+            _ptr(a_bias), _ptr(u_bias), c_int(width), _ptr(seqs), c_int(n_seqs), c_int(int(single_tokens)), _ptr(state),
+            c_long(state.stride(0)), _ptr(out), c_long(out.stride(0)), _stream()))
+
+    def embed_positions(self, tokens: torch.Tensor, tok_pos, table: torch.Tensor, freq: torch.Tensor, out: torch.Tensor,
+                        scale: float = 1.0) -> None:
+        """``out[t] = table[tokens[t]] * scale + v`` as float32 rows, ``v[2i] = sin(p freq[i])`` and ``v[2i + 1] = cos(p
+        freq[i])`` at the token's position ``p``; ``freq`` float64 ``[(width + 1) // 2]``."""
+        _rows_ok(table, "embed_positions table"); _rows_ok(out, "embed_positions out")
+        t, width = out.shape
+        for name, v in (("tokens", tokens), ("tok_pos", tok_pos)):
+            if not (v.is_cuda and v.dtype == torch.int32 and v.dim() == 1 and v.is_contiguous() and v.shape[0] >= t):
+                raise KernelError(f"embed_positions {name}: a contiguous int32 vector on the GPU, one entry a token")
+        if not (table.is_contiguous() and table.dtype in DTYPE_CODE and table.shape[1] == width and out.dtype == torch.float32):
+            raise KernelError("embed_positions: a contiguous float32/bfloat16 table and float32 rows of its width")
+        if not (freq.is_cuda and freq.dtype == torch.float64 and freq.is_contiguous() and freq.numel() == (width + 1) // 2):
+            raise KernelError(f"embed_positions freq must be float64 with {(width + 1) // 2} elements on the GPU")
+        if t == 0:
+            return
+        lib = self.mixers_lib()
+        self._launch(lib, lib.ls_embed_positions, (
+            c_int(DTYPE_CODE[table.dtype]), _ptr(tokens), _ptr(tok_pos), _ptr(table), c_int(table.shape[0]), _ptr(freq),
+            _ptr(out), c_int(t), c_int(width), c_long(out.stride(0)), c_float(scale), _stream()))
 
 
 ATTENTION_ITEM_INTS = 32

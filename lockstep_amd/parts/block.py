@@ -157,6 +157,19 @@ class PreNormResidual(Arrangement):
         return left if isinstance(left, PendingAdd) else None
 
 
+def as_slices(ctx, name: str, defers: bool, call, width: int):
+    """One sublayer's output as slice sums ``[slices, T, width]``.  ``call(out, accumulate, defer)`` runs the sublayer."""
+    import torch
+
+    t = ctx.n_tokens
+    y = ctx.buf(name, (t, width), torch.float32)
+    # (a part that defers leaves slice sums and does not touch y; else it stores its output there)
+    left = call(y, False, "any") if defers else call(y, False, False)
+    if isinstance(left, PendingAdd):
+        return left.partials
+    return y.view(1, t, width)
+
+
 class PendingWrite(PendingAdd):
     """A sublayer's output that still has to be written into a residual stream of several copies:
     ``x'_t = sum_s mix[s, t] x_s + gain[t] y`` with ``y`` the sum of ``partials`` in ascending order.
@@ -263,18 +276,6 @@ class HyperConnections(Arrangement):
             full = self.join(self.layer_spec.prefix, name)
             self.streams[sublayer] = tuple(rt.vector(weights.get(f"{full}.{t}").reshape(-1)) for t in ("in", "out", "mix"))
 
-    def _run(self, ctx, sublayer, defers: bool, call, width: int):
-        """One sublayer's output as slice sums ``[slices, T, width]``."""
-        import torch
-
-        t = ctx.n_tokens
-        y = ctx.buf(f"streams.y.{sublayer}", (t, width), torch.float32)
-        # (a part that defers leaves slice sums and does not touch y; else it stores its output there)
-        left = call(y, False, "any") if defers else call(y, False, False)
-        if isinstance(left, PendingAdd):
-            return left.partials
-        return y.view(1, t, width)
-
     def forward(self, ctx, run, h, pending=None):
         """``pending``: the write the previous layer left (a ``PendingWrite``).  Returns this layer's last one."""
         rt = ctx.rt
@@ -292,7 +293,7 @@ class HyperConnections(Arrangement):
             call = lambda y, acc, defer: self._mixer.forward(ctx, run, x, y, accumulate=acc, defer=defer)  # noqa: E731
         else:
             call = lambda y, acc, defer: self._mixer.forward(ctx, run, x, y, accumulate=acc)  # noqa: E731
-        left = PendingWrite(self._run(ctx, "mixer", self._defer_mixer, call, width), mix, gain, n)
+        left = PendingWrite(as_slices(ctx, "streams.y.mixer", self._defer_mixer, call, width), mix, gain, n)
         if self.feed_forward is None:
             return left
         take, gain, mix = self.streams["feed_forward"]
@@ -303,4 +304,136 @@ class HyperConnections(Arrangement):
             call = lambda y, acc, defer: self.feed_forward.forward(ctx, x, y, accumulate=acc, defer=defer)  # noqa: E731
         else:
             call = lambda y, acc, defer: self.feed_forward.forward(ctx, x, y, accumulate=acc)  # noqa: E731
-        return PendingWrite(self._run(ctx, "feed_forward", self._defer_ff, call, width), mix, gain, n)
+        return PendingWrite(as_slices(ctx, "streams.y.feed_forward", self._defer_ff, call, width), mix, gain, n)
+
+
+class PendingStep(PendingAdd):
+    """What is still to be done to the residual stream behind a sublayer with a norm of its output: ``x += norm(y)``
+    with ``y`` the sum of ``partials`` in ascending order (``post``: (weight, eps, centred); None: ``x += y``); then, at a
+    layer's end with an average over depth, ``results[keep] = x`` and ``x = sum_j shares[j] results[j]``.  The next
+    reader of the stream (a norm) does it on its way, in one launch."""
+
+    def __init__(self, partials, post, results=None, keep: int = 0, shares=None):
+        super().__init__(partials)
+        self.post, self.results, self.keep, self.shares = post, results, keep, shares
+
+    def step(self, ctx, stream, norm, out, rows=None) -> None:
+        """The pending work, then ``out = norm(x)``; with ``rows`` only those rows are read, and only ``out`` is written."""
+        ctx.rt.kernels.residual_step(stream, self.partials, self.post, self.results, self.keep, self.shares, norm, out, rows)
+
+    def flush(self, ctx, stream, rows=None) -> None:
+        if rows is not None:
+            raise ValueError("the step behind a sublayer is flushed for all rows")
+        self.step(ctx, stream, None, None)
+
+
+@register_part("sandwich_residual")
+class SandwichResidual(Arrangement):
+    """A norm in front of each sublayer and one behind it: ``x += post_1(mixer(norm_1(x)))``; ``x +=
+    post_2(feed_forward(norm_2(x)))``.  A layer without a ``feed_forward`` part is the first half alone.
+
+    Parts of the layer: ``mixer``, ``mixer_norm``, ``mixer_post_norm``, and ``feed_forward``, ``feed_forward_norm``,
+    ``feed_forward_post_norm``; the norms are ``layernorm`` or ``rmsnorm`` parts.  Parameters: ``mixer_prefix``,
+    ``feed_forward_prefix``, and the norms' tensor names below the layer's prefix, ``mixer_norm_name``,
+    ``mixer_post_norm_name``, ``feed_forward_norm_name``, ``feed_forward_post_norm_name``.
+
+    ``depth_average`` (optional, ``{"name", "index", "layers"}``): with ``X_0`` the embedding's output and ``X_(i+1)`` what
+    layer ``i`` leaves, layer ``i`` (``index``, of ``layers``) hands on ``sum_j a[j] X_j`` over ``j = 0 .. i+1`` with the
+    tensor ``a [index + 2]``.  The results of a step's tokens stay in a buffer of the step, ``[layers + 1, T, width]``
+    float32; nothing of it is kept between steps.
+
+    The addition of a sublayer's normed output, the average and the next sublayer's norm are one launch
+    (``PendingStep``)."""
+
+    graph_safe = True
+
+    NORMS = ("mixer_norm", "mixer_post_norm", "feed_forward_norm", "feed_forward_post_norm")
+
+    def __init__(self, layer_spec, prefix: str = ""):
+        super().__init__(layer_spec, build_part)
+        p = layer_spec.arrangement.params
+        base = layer_spec.prefix
+        build = lambda name: build_part(layer_spec.part(name), self.join(base, p[f"{name}_name"]))  # noqa: E731
+        self._mixer = build_part(layer_spec.part("mixer"), self.join(base, p["mixer_prefix"]))
+        self.mixer_norm, self.mixer_post_norm = build("mixer_norm"), build("mixer_post_norm")
+        self.feed_forward = self.feed_forward_norm = self.feed_forward_post_norm = None
+        if layer_spec.has("feed_forward"):
+            self.feed_forward = build_part(layer_spec.part("feed_forward"), self.join(base, p["feed_forward_prefix"]))
+            self.feed_forward_norm, self.feed_forward_post_norm = build("feed_forward_norm"), build("feed_forward_post_norm")
+        for norm in self.parts():
+            if norm not in (self._mixer, self.feed_forward) and not hasattr(norm, "step_norm"):
+                raise ValueError(f"{norm.kind!r} norms cannot stand around a sublayer of this arrangement")
+        self._defer_mixer = takes(self._mixer.forward, "defer")
+        self._defer_ff = self.feed_forward is not None and takes(self.feed_forward.forward, "defer")
+        self.depth = p.get("depth_average")
+        self.shares = None
+        if self.depth is not None and not 0 <= int(self.depth["index"]) < int(self.depth["layers"]):
+            raise ValueError(f"layer {self.depth['index']} of {self.depth['layers']} in an average over depth")
+
+    @classmethod
+    def weight_specs(cls, layer_spec, prefix: str = ""):
+        from .base import part_class
+
+        p = layer_spec.arrangement.params
+        base = layer_spec.prefix
+        out = []
+        # (a norm the checkpoint may hold although nothing follows it is an optional part: accepted, never used)
+        for name in ("mixer", "feed_forward") + cls.NORMS:
+            if layer_spec.has(name):
+                spec = layer_spec.part(name)
+                key = p[f"{name}_name"] if name in cls.NORMS else p[f"{name}_prefix"]
+                out += part_class(spec.kind).weight_specs(spec, cls.join(base, key))
+        depth = p.get("depth_average")
+        if depth is not None:
+            out.append(WeightSpec(cls.join(base, depth["name"]), (int(depth["index"]) + 2,), kind="vector", init="unit"))
+        return out
+
+    def parts(self):
+        mine = (self._mixer, self.mixer_norm, self.mixer_post_norm)
+        if self.feed_forward is None:
+            return mine
+        return mine + (self.feed_forward, self.feed_forward_norm, self.feed_forward_post_norm)
+
+    @property
+    def mixer(self):
+        return self._mixer
+
+    def load(self, weights, rt) -> None:
+        for part in self.parts():
+            part.load(weights, rt)
+        if self.depth is not None:
+            self.shares = rt.vector(weights.get(self.join(self.layer_spec.prefix, self.depth["name"])))
+        rt.kernels.mixers_lib()
+
+    def forward(self, ctx, run, h, pending=None):
+        """``pending``: what the previous layer left to do.  Returns what this layer leaves (a ``PendingStep``)."""
+        import torch
+
+        k = ctx.rt.kernels
+        t, width = ctx.n_tokens, h.shape[1]
+        results, index = None, 0
+        if self.depth is not None:
+            layers, index = int(self.depth["layers"]), int(self.depth["index"])
+            results = ctx.buf("depth.results", ((layers + 1) * t, width), torch.float32).view(layers + 1, t, width)
+        x = ctx.buf("block.normed", (t, width), ctx.rt.dtype)
+        if pending is not None and not isinstance(pending, PendingStep):
+            pending.flush(ctx, h)
+            pending = None
+        if pending is not None:
+            pending.step(ctx, h, self.mixer_norm.step_norm(), x)
+        else:                                     # (the first layer also keeps what it finds in the stream)
+            k.residual_step(h, None, None, results if index == 0 else None, 0, None, self.mixer_norm.step_norm(), x)
+        if self._defer_mixer:
+            call = lambda y, acc, defer: self._mixer.forward(ctx, run, x, y, accumulate=acc, defer=defer)  # noqa: E731
+        else:
+            call = lambda y, acc, defer: self._mixer.forward(ctx, run, x, y, accumulate=acc)  # noqa: E731
+        y = as_slices(ctx, "sandwich.y.mixer", self._defer_mixer, call, width)
+        if self.feed_forward is None:
+            return PendingStep(y, self.mixer_post_norm.step_norm(), results, index + 1, self.shares)
+        k.residual_step(h, y, self.mixer_post_norm.step_norm(), None, 0, None, self.feed_forward_norm.step_norm(), x)
+        if self._defer_ff:
+            call = lambda y, acc, defer: self.feed_forward.forward(ctx, x, y, accumulate=acc, defer=defer)  # noqa: E731
+        else:
+            call = lambda y, acc, defer: self.feed_forward.forward(ctx, x, y, accumulate=acc)  # noqa: E731
+        y = as_slices(ctx, "sandwich.y.feed_forward", self._defer_ff, call, width)
+        return PendingStep(y, self.feed_forward_post_norm.step_norm(), results, index + 1, self.shares)

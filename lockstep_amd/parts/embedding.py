@@ -2,6 +2,8 @@
 
 from __future__ import annotations
 
+import torch
+
 from ..config.base import PartSpec
 from ..ops import STORE_F32
 from .base import Part, StateSpec, WeightSpec, register_part
@@ -17,7 +19,10 @@ class TokenEmbedding(Part):
     ``pairs`` (optional, ``{"name", "buckets", "mul_prev", "mul_cur"}``): a second table ``[buckets + 1,
     hidden_size]`` is added, row ``(token before * mul_prev + token * mul_cur) mod buckets``, and its last
     row for a request's first token.  The token before a step's first one is kept per request (one int:
-    the part then has a ``state_spec`` and the model names a cache unit for it)."""
+    the part then has a ``state_spec`` and the model names a cache unit for it).
+
+    ``positions`` (optional, ``{"base"}``): a vector of sines and cosines of the token's position is added,
+    ``sin(p * base^(-2i/hidden_size))`` to element ``2i`` and the cosine to element ``2i + 1``."""
 
     graph_safe = True
     state_unit = None       # the cache unit of the kept token, set by the model
@@ -28,6 +33,13 @@ class TokenEmbedding(Part):
         self.scale = float(spec.params.get("scale", 1.0))
         self.copies = int(spec.params.get("copies") or 1)
         self.pairs = spec.params.get("pairs")
+        self.positions = spec.params.get("positions")
+        self.frequencies = None
+        if self.positions is not None:
+            if self.copies != 1 or self.pairs is not None:
+                raise ValueError("an embedding with position vectors fills one copy of the stream and has no table of pairs")
+            if not float(self.positions["base"]) > 0:
+                raise ValueError(f"the base of the position vectors must be positive, got {self.positions['base']!r}")
         if self.pairs is not None:
             if self.copies != 1:
                 raise ValueError("an embedding with a table of pairs fills one copy of the stream")
@@ -50,8 +62,16 @@ class TokenEmbedding(Part):
         if self.pairs is not None:
             self.pair_table = rt.matrix(weights.get(self.pairs["name"]))
             rt.kernels.mixers_lib()
+        if self.positions is not None:
+            width, base = int(self.spec["hidden_size"]), float(self.positions["base"])
+            self.frequencies = torch.tensor([base ** (-2.0 * i / width) for i in range((width + 1) // 2)],
+                                            dtype=torch.float64, device=rt.device)
+            rt.kernels.mixers_lib()
 
     def forward(self, ctx, tokens, out) -> None:
+        if self.positions is not None:
+            ctx.rt.kernels.embed_positions(tokens, ctx.tok_pos, self.table, self.frequencies, out, self.scale)
+            return
         if self.pairs is None:
             ctx.rt.kernels.embed(tokens, self.table, out, self.scale, self.copies)
             return

@@ -100,6 +100,65 @@ class GatedMLP(FeedForward):
         return None
 
 
+@register_part("mlp")
+class MLP(FeedForward):
+    """``down(act(up(x)))``: a feed-forward of two matrices.  Parameters: ``hidden_size``, ``intermediate_size``,
+    ``activation`` (``xielu``, or ``silu``, ``gelu``, ``gelu_tanh``, ``relu``), and optionally the tensor names below the
+    prefix ``up_name``, ``down_name`` (default ``up``, ``down``) and, for ``xielu``, ``act_name`` (default ``act``).
+
+    ``xielu`` has two learned numbers (p, q): ``softplus(p) z^2 + z/2`` above zero, ``(1/2 + softplus(q)) (e^z - 1 - z) +
+    z/2`` elsewhere.  It is the up product's epilogue; the softplus of both numbers is taken once, at load.  The other
+    activations store the up product in float32 and run as a pass of their own."""
+
+    graph_safe = True
+    repeatable = True
+
+    def __init__(self, spec: PartSpec, prefix: str = ""):
+        super().__init__(spec, prefix)
+        self.hidden = int(spec["hidden_size"])
+        self.inter = int(spec["intermediate_size"])
+        self.activation = str(spec["activation"])
+        if self.activation not in ("xielu", "silu", "gelu", "gelu_tanh", "relu"):
+            raise ValueError(f"activation {self.activation!r} is not built; known: xielu, silu, gelu, gelu_tanh, relu")
+        self.w_up = self.w_down = self.factors = None
+
+    @classmethod
+    def names(cls, spec: PartSpec, prefix: str):
+        return tuple(f"{prefix}.{spec.params.get(key, default)}" for key, default in
+                     (("up_name", "up"), ("down_name", "down"), ("act_name", "act")))
+
+    @classmethod
+    def weight_specs(cls, spec: PartSpec, prefix: str) -> list[WeightSpec]:
+        h, i = int(spec["hidden_size"]), int(spec["intermediate_size"])
+        up, down, act = cls.names(spec, prefix)
+        out = [WeightSpec(up, (i, h)), WeightSpec(down, (h, i))]
+        if spec["activation"] == "xielu":
+            out.append(WeightSpec(act, (2,), kind="vector"))
+        return out
+
+    def load(self, weights, rt) -> None:
+        up, down, act = self.names(self.spec, self.prefix)
+        self.w_up = rt.matrix(weights.get(up))
+        self.w_down = rt.matrix(weights.get(down))
+        if self.activation == "xielu":
+            both = torch.nn.functional.softplus(weights.get(act).to(torch.float64).reshape(2), threshold=40.0)
+            self.factors = rt.vector((both + torch.tensor([0.0, 0.5], dtype=torch.float64)).to(torch.float32))
+
+    def forward(self, ctx, x, out, accumulate: bool, defer: bool = False):
+        from .base import project_out
+
+        rt = ctx.rt
+        k = rt.kernels
+        act = ctx.buf("mlp.act", (ctx.n_tokens, self.inter), rt.dtype)
+        if self.activation == "xielu":
+            k.gemm_xielu(x, self.w_up, act, self.factors)
+        else:
+            wide = ctx.buf("mlp.up", (ctx.n_tokens, self.inter), torch.float32)
+            k.gemm(x, self.w_up, wide, STORE_F32)
+            k.bias_act(wide, None, act, self.activation)
+        return project_out(ctx, act, self.w_down, out, accumulate, defer, "mlp.down_slices")
+
+
 @register_part("clamped_gated_mlp")
 class ClampedGatedMLP(FeedForward):
     """``down(g * sigmoid(alpha * g) * (u + 1))`` with ``g = min(gate(x), limit)`` and ``u = clamp(up(x),

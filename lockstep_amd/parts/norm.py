@@ -1,5 +1,5 @@
 """Norms of the residual stream.  RMSNorm: ``y = x * 1/sqrt(mean(x^2) + eps) * w`` in 32-bit
-(reference engine/kernels/rmsnorm.py:30-38).  Dynamic Tanh: ``y = tanh(alpha x) * w + b``, which
+(reference engine/kernels/rmsnorm.py:30-38).  Layer norm: the same of the deviations from the row's mean.  Dynamic Tanh: ``y = tanh(alpha x) * w + b``, which
 takes no statistics of the row."""
 
 from __future__ import annotations
@@ -47,6 +47,11 @@ class RMSNorm(Norm):
 
     def forward(self, ctx, x, out, rows=None, pending=None) -> None:
         """``pending`` (a ``PendingAdd``): added to ``x`` first, in the same launch."""
+        if hasattr(pending, "post"):
+            if self.copies > 1:
+                raise ValueError("a stream of several copies takes the pending write of its own arrangement only")
+            pending.step(ctx, x, self.step_norm(), out, rows)
+            return
         if self.copies > 1 or hasattr(pending, "mix"):
             # the sum of the copies, after what the last sublayer still has to write into them
             if pending is not None and not hasattr(pending, "mix"):
@@ -59,6 +64,57 @@ class RMSNorm(Norm):
             ctx.rt.kernels.add_rmsnorm(x, pending.partials, self.weight, out, self.eps, rows)
         else:
             ctx.rt.kernels.rmsnorm(x, self.weight, out, self.eps, rows)
+
+
+    def step_norm(self):
+        """The norm as ``Kernels.residual_step`` takes it: (weight, eps, whether the mean is subtracted)."""
+        return self.weight, self.eps, False
+
+
+@register_part("layernorm")
+class LayerNorm(Norm):
+    """``y = (x - mean) / sqrt(mean((x - mean)^2) + eps) * w`` in 32-bit, no bias.  Parameters: ``size``, ``eps``; ``name``
+    overrides the tensor name (default: the prefix itself).  With ``optional`` the weight may be absent (a layer whose
+    second half is missing never runs the norm)."""
+
+    graph_safe = True
+    repeatable = True
+
+    def __init__(self, spec: PartSpec, prefix: str = ""):
+        super().__init__(spec, prefix)
+        self.size = int(spec["size"])
+        self.eps = float(spec["eps"])
+        self.weight = None
+
+    @staticmethod
+    def tensor_name(spec: PartSpec, prefix: str) -> str:
+        return spec.params.get("name") or prefix
+
+    @classmethod
+    def weight_specs(cls, spec: PartSpec, prefix: str) -> list[WeightSpec]:
+        return [WeightSpec(cls.tensor_name(spec, prefix), (int(spec["size"]),), kind="vector", init="norm",
+                           optional=bool(spec.params.get("optional")))]
+
+    def load(self, weights, rt) -> None:
+        name = self.tensor_name(self.spec, self.prefix)
+        if self.spec.params.get("optional") and name not in weights:
+            return
+        self.weight = rt.vector(weights.get(name))
+        rt.kernels.mixers_lib()
+
+    def step_norm(self):
+        """The norm as ``Kernels.residual_step`` takes it: (weight, eps, whether the mean is subtracted)."""
+        return self.weight, self.eps, True
+
+    def forward(self, ctx, x, out, rows=None, pending=None) -> None:
+        """``pending`` (a ``PendingAdd``): added to ``x`` first, in the same launch."""
+        if hasattr(pending, "mix"):
+            raise ValueError("layernorm does not read a residual stream of several copies")
+        if hasattr(pending, "post"):
+            pending.step(ctx, x, self.step_norm(), out, rows)
+            return
+        ctx.rt.kernels.residual_step(x, None if pending is None else pending.partials, None, None, 0, None, self.step_norm(),
+                                     out, rows)
 
 
 @register_part("dynamic_tanh")

@@ -1,6 +1,6 @@
 """Linear-attention mixers that keep a matrix of fixed size per request and head instead of keys
-and values.  ``gated_delta`` (at the end of this file) is the delta rule with a decay a head and short
-convolutions in front; the two others share one recurrence with a decay and a write gate for every row of the state,
+and values.  ``gated_delta`` (below) is the delta rule with a decay a head and short
+convolutions in front; ``min_gru`` (at the end of this file) keeps one number a channel; the two others share one recurrence with a decay and a write gate for every row of the state,
 
     S_t = diag(a_t) S_(t-1) + b_t v_t^T          S [dim, vdim] in float32, zero at the start
     o_t = S_t^T q_t
@@ -298,3 +298,60 @@ class GatedDelta(Mixer):
         gated = ctx.buf("delta.normed", (t, n * dv), rt.dtype)
         k.head_norm_gate(o, n, dv, self.norm, gate, self.eps, gated, gate_act=self.gate_act)
         return project_out(ctx, gated, self.w_o, out, accumulate, defer, "delta.out_slices")
+
+
+@register_part("min_gru")
+class MinGRU(Mixer):
+    """A gated recurrence of one number a channel whose gates read the current token only:
+
+        z = sigmoid(W_z h + b_z);  v = W_x h + b_x;  c = v + 1/2 where v >= 0, else sigmoid(v)
+        S_t = (1 - z) S_(t-1) + z c          S [state_size] in float32, zero at the start
+        out = W_o (S_t * silu(W_g h))
+
+    Parameters: ``hidden_size``, ``state_size``.  Tensors below the prefix: ``z``, ``x``, ``g`` ``[state_size, hidden]``,
+    ``z.b``, ``x.b`` ``[state_size]``, ``o`` ``[hidden, state_size]``.
+
+    The three projections are one matrix product stored in float32; gates, candidate, recurrence and output gate are one
+    launch in 32-bit that leaves what ``W_o`` reads."""
+
+    graph_safe = True
+    repeatable = True
+
+    def __init__(self, spec: PartSpec, prefix: str = ""):
+        super().__init__(spec, prefix)
+        self.hidden, self.size = int(spec["hidden_size"]), int(spec["state_size"])
+        if min(self.hidden, self.size) <= 0:
+            raise ValueError("the sizes of a recurrent mixer must be positive")
+        self.w_in = self.w_o = self.z_bias = self.x_bias = None
+
+    @classmethod
+    def weight_specs(cls, spec: PartSpec, prefix: str) -> list[WeightSpec]:
+        h, w = int(spec["hidden_size"]), int(spec["state_size"])
+        return [WeightSpec(f"{prefix}.z", (w, h)), WeightSpec(f"{prefix}.z.b", (w,), kind="vector"),
+                WeightSpec(f"{prefix}.x", (w, h)), WeightSpec(f"{prefix}.x.b", (w,), kind="vector"),
+                WeightSpec(f"{prefix}.g", (w, h)), WeightSpec(f"{prefix}.o", (h, w))]
+
+    def cache_spec(self):
+        return StateSpec((self.size,), "float32")
+
+    def mixing_flops(self, tokens: int, start: int) -> float:
+        return 3.0 * self.size * tokens
+
+    def load(self, weights, rt) -> None:
+        tensors = [weights.get(f"{self.prefix}.{n}") for n in "zxg"]
+        if len({t.dtype for t in tensors}) > 1:
+            tensors = [t.to(torch.float32) for t in tensors]
+        self.w_in = rt.matrix(torch.cat(tensors, dim=0))
+        self.w_o = rt.matrix(weights.get(f"{self.prefix}.o"))
+        self.z_bias = rt.vector(weights.get(f"{self.prefix}.z.b"))
+        self.x_bias = rt.vector(weights.get(f"{self.prefix}.x.b"))
+        rt.kernels.mixers_lib()
+
+    def forward(self, ctx, run, x, out, accumulate: bool, defer: bool = False):
+        rt, k, t, w = ctx.rt, ctx.rt.kernels, ctx.n_tokens, self.size
+        raw = ctx.buf("recurrence.in_f32", (t, 3 * w), torch.float32)
+        k.gemm(x, self.w_in, raw, STORE_F32)
+        gated = ctx.buf("recurrence.normed", (t, w), rt.dtype)
+        k.channel_recurrence(raw, 0, w, 2 * w, self.z_bias, self.x_bias, ctx.seqs, ctx.n_seqs, ctx.single_tokens,
+                             ctx.cache.unit_state(run.cache), gated)
+        return project_out(ctx, gated, self.w_o, out, accumulate, defer, "recurrence.out_slices")
