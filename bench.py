@@ -448,6 +448,27 @@ def narurax_like(qwen, layers: int, window: int = 4096, keep_first: int = 4, exp
                              "layers": [cycle[i % 4] for i in range(layers)]})
 
 
+def tukavik_like(qwen, layers: int):
+    """A Tukavik configuration at the layer sizes of the Qwen3 configuration ``qwen``: the layers cycle through the
+    recurrence of one number a channel (as many channels as the Qwen3 attention's heads have elements), attention over a
+    latent, the same with queries through a latent of their own, and the last reading the latent of the layer before;
+    the attention has the heads and head size of the Qwen3 attention (the latent: as many elements as a head, the query
+    latent three times that).  The feed-forward's two matrices multiply as much as Qwen3's three."""
+    from lockstep_amd.config import config_from_dict
+
+    heads, d = qwen.num_attention_heads, qwen.head_dim
+    mlp = {"kind": "dense", "ff": qwen.intermediate_size * 3 // 2}
+    plain = {"heads": heads, "dim": d, "vdim": d, "kv_rank": d, "scale": d ** -0.5}
+    through = dict(plain, q_rank=3 * d)
+    out = []
+    for i in range(layers):
+        kind, mixer = [("mingru", {"width": heads * d}), ("latent_attention", plain), ("latent_attention_2", through),
+                       ("latent_attention_2", dict(through, kv_from=i - 1))][i % 4]
+        out.append({"type": kind, "mixer": mixer, "mlp": mlp})
+    return config_from_dict({"architecture": "Tukavik", "vocab": qwen.vocab_size, "width": qwen.hidden_size,
+                             "norm": {"eps": qwen.rms_norm_eps}, "layers": out})
+
+
 def designs_record(args) -> dict:
     """Prefill and decode of the other designs beside Qwen3 at equal layer sizes."""
     import gc
@@ -466,7 +487,8 @@ def designs_record(args) -> dict:
            "prefill_tokens": args.prefill_len, "prompt_len": args.prompt_len, "steps": args.steps,
            "data": "synthetic: uniform random token ids, random weights", "designs": {}}
     makers = {"qwen3": lambda: qwen, "bikovik": lambda: bikovik_like(qwen, layers), "biberax": lambda: biberax_like(qwen, layers),
-              "toripel": lambda: toripel_like(qwen, layers), "narurax": lambda: narurax_like(qwen, layers)}
+              "toripel": lambda: toripel_like(qwen, layers), "narurax": lambda: narurax_like(qwen, layers),
+              "tukavik": lambda: tukavik_like(qwen, layers)}
     for name in args.designs.split(","):
         if name not in makers:
             raise SystemExit(f"--designs: {name!r} is not one of {', '.join(makers)}")
@@ -646,7 +668,7 @@ def main(argv=None) -> int:
                         "scheduler; contexts: prefill and decode at the context lengths of --contexts; designs: "
                         "the Bikovik and Biberax designs beside Qwen3 at the layer sizes of --model")
     p.add_argument("--contexts", default="4096,8192,16384", help="contexts: the context lengths, comma separated")
-    p.add_argument("--designs", default="qwen3,bikovik,biberax", help="designs: which of qwen3, bikovik, biberax, toripel, narurax, comma separated")
+    p.add_argument("--designs", default="qwen3,bikovik,biberax", help="designs: which of qwen3, bikovik, biberax, toripel, narurax, tukavik, comma separated")
     p.add_argument("--repeats", type=int, default=5, help="timed runs; the median is reported with the spread")
     p.add_argument("--requests", type=int, default=0, help="serve: only the first N requests of the workload")
     p.add_argument("--prefill-chunk", type=int, default=None, help="serve: prompt portion (0: whole prompts)")

@@ -142,20 +142,43 @@ __device__ __forceinline__ void epilogue_swiglu4(void* __restrict__ C, long ldc,
   epilogue4<T, kStore>(C, ldc, m, col, M, width, act, vec_ok);
 }
 
+// e^z - 1 - z for z <= 0.  Near zero the three terms cancel: the library's e^z - 1 on the 32-bit path; in front of a
+// rounding to bfloat16 the series z^2/2 (1 + z/3 (1 + z/4 (...))) down to -1/2 (its first missing term is below 2e-6 of
+// the sum) and the hardware's exponential beyond.
+template <typename T> __device__ __forceinline__ float exp_beyond_linear(float z);
+template <> __device__ __forceinline__ float exp_beyond_linear<float>(float z) { return expm1f(z) - z; }
+template <> __device__ __forceinline__ float exp_beyond_linear<bf16_t>(float z) {
+  float s = fmaf(z, 1.0f / 7.0f, 1.0f);
+  s = fmaf(z * (1.0f / 6.0f), s, 1.0f);
+  s = fmaf(z * (1.0f / 5.0f), s, 1.0f);
+  s = fmaf(z * (1.0f / 4.0f), s, 1.0f);
+  s = fmaf(z * (1.0f / 3.0f), s, 1.0f);
+  return z > -0.5f ? 0.5f * z * z * s : (__expf(z) - 1.0f) - z;
+}
+
 // xIELU of a float total:  up z^2 + z/2 above zero,  down (e^z - 1 - z) + z/2 elsewhere.
+template <typename T>
 __device__ __forceinline__ float xielu(float z, float up, float down) {
-  const float low = fminf(z, 0.f);
-  return (z > 0.f ? up * (z * z) : down * (expm1f(low) - low)) + 0.5f * z;
+  return (z > 0.f ? up * (z * z) : down * exp_beyond_linear<T>(fminf(z, 0.f))) + 0.5f * z;
+}
+
+// The activation's two factors, asked for when a kernel starts (they are needed when it ends).
+struct Factors {
+  float up, down;
+};
+template <int EPI>
+__device__ __forceinline__ Factors load_factors(const float* __restrict__ act) {
+  if constexpr (EPI == kXielu) return Factors{act[0], act[1]};
+  return Factors{0.f, 0.f};
 }
 
 template <typename T>
 __device__ __forceinline__ void epilogue_xielu4(void* __restrict__ C, long ldc, int m, int n, int M, int N,
-                                                const float total[4], bool vec_ok, const float* __restrict__ act) {
+                                                const float total[4], bool vec_ok, const Factors& factors) {
   if (m >= M || n >= N) return;
-  const float up = act[0], down = act[1];
   float v[4];
 #pragma unroll
-  for (int r = 0; r < 4; ++r) v[r] = xielu(total[r], up, down);
+  for (int r = 0; r < 4; ++r) v[r] = xielu<T>(total[r], factors.up, factors.down);
   epilogue4<T, kStore>(C, ldc, m, n, M, N, v, vec_ok);
 }
 
@@ -207,6 +230,7 @@ __global__ __launch_bounds__(NW * 64) void gemm_skinny_kernel(const void* __rest
   typedef Atom<T> A;
   typedef typename A::vec_t vec_t;
   constexpr int NT = (EPI == kSwiGLU) ? 2 : 1;  // weight tiles per workgroup
+  const Factors factors = load_factors<EPI>(act);
   extern __shared__ float part[];                // [nslices][NT][MT][256] (+ 80 floats with NORM)
 
   const int lane = threadIdx.x & 63;
@@ -338,7 +362,7 @@ __global__ __launch_bounds__(NW * 64) void gemm_skinny_kernel(const void* __rest
     if (EPI == kSwiGLU)
       epilogue_swiglu4<T>(C, ldc, m, blockIdx.x * 16 + (l >> 4) * 4, M, out_cols, total[0], total[NT - 1], vec_ok);
     else if constexpr (EPI == kXielu)
-      epilogue_xielu4<T>(C, ldc, m, n0 + (l >> 4) * 4, M, N, total[0], vec_ok, act);
+      epilogue_xielu4<T>(C, ldc, m, n0 + (l >> 4) * 4, M, N, total[0], vec_ok, factors);
     else
       epilogue4<T, EPI>(C, ldc, m, n0 + (l >> 4) * 4, M, N, total[0], vec_ok,
                         (preload && idx == (int)threadIdx.x) ? &old_vals : nullptr);
@@ -366,6 +390,7 @@ __global__ __launch_bounds__(1024) void gemm_stream_kernel(const T* __restrict__
   typedef Atom<T> A;
   typedef typename A::vec_t vec_t;
   constexpr int NT = (EPI == kSwiGLU) ? 2 : 1;  // weight tiles per column block
+  const Factors factors = load_factors<EPI>(act);
   constexpr int UC = 4;                          // chunks per unit
   constexpr int UQ = XC / UC;                    // units per tile
   constexpr int UNITS = NT * UQ;                 // units per column block
@@ -473,7 +498,7 @@ __global__ __launch_bounds__(1024) void gemm_stream_kernel(const T* __restrict__
       if (EPI == kSwiGLU)
         epilogue_swiglu4<T>(C, ldc, m, b * 16 + g * 4, M, out_cols, total[0], total[NT - 1], vec_ok);
       else if constexpr (EPI == kXielu)
-        epilogue_xielu4<T>(C, ldc, m, b * 16 + g * 4, M, N, total[0], vec_ok, act);
+        epilogue_xielu4<T>(C, ldc, m, b * 16 + g * 4, M, N, total[0], vec_ok, factors);
       else
         epilogue4<T, EPI>(C, ldc, m, b * 16 + g * 4, M, N, total[0], vec_ok);
     }
@@ -893,6 +918,7 @@ __global__ __launch_bounds__(64 * NWM * NWN) void gemm_tiled_kernel(const T* __r
                                                          int out_cols, const float* __restrict__ act) {
   typedef Atom<T> A;
   typedef typename A::vec_t vec_t;
+  const Factors factors = load_factors<EPI>(act);
   constexpr int BK = kRowBytes / sizeof(T);  // elements of K per stage
   constexpr int TI = BN / (16 * NWN);        // weight tiles (16 columns) per wave
   constexpr int TJ = BM / (16 * NWM);        // row tiles per wave
@@ -1099,7 +1125,7 @@ __global__ __launch_bounds__(64 * NWM * NWN) void gemm_tiled_kernel(const T* __r
       for (int j = 0; j < TJ; ++j) {
         float t[4] = {total[i][j][0], total[i][j][1], total[i][j][2], total[i][j][3]};
         if constexpr (EPI == kXielu)
-          epilogue_xielu4<T>(C, ldc, m_base + wm + j * 16 + row16, n_base + wn + i * 16 + g * 4, M, N, t, vec_ok, act);
+          epilogue_xielu4<T>(C, ldc, m_base + wm + j * 16 + row16, n_base + wn + i * 16 + g * 4, M, N, t, vec_ok, factors);
         else
           epilogue4<T, EPI>(C, ldc, m_base + wm + j * 16 + row16, n_base + wn + i * 16 + g * 4, M, N, t, vec_ok);
       }

@@ -244,7 +244,8 @@ __global__ __launch_bounds__(256) void latent_query_kernel(const float* __restri
 template <typename T, int RT>
 __global__ __launch_bounds__(256) void heads_product_kernel(const T* __restrict__ x, long ldx, int x_stride,
                                                             const T* __restrict__ w, int N, int K, int n_rows,
-                                                            T* __restrict__ out, long ldo, int o_stride, int x_aligned) {
+                                                            T* __restrict__ out, long ldo, int o_stride, int x_aligned,
+                                                            int out_vec) {
   constexpr int VEC = Atom<T>::VEC, KC = Atom<T>::KCHUNK;
   const int head = blockIdx.y;
   const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6;
@@ -284,6 +285,14 @@ __global__ __launch_bounds__(256) void heads_product_kernel(const T* __restrict_
   for (int r = 0; r < RT; ++r) {
     if (!x_ok[r]) continue;
     T* dst = out + (long)(row0 + 16 * r + l16) * ldo + (long)head * o_stride;
+    if (out_vec && col0 + 4 * quad + 3 < N) {   // a lane's four columns in one store
+      typedef T out4 __attribute__((ext_vector_type(4)));
+      out4 v;
+#pragma unroll
+      for (int i = 0; i < 4; ++i) v[i] = from_f32<T>(acc[r][i]);
+      *reinterpret_cast<out4*>(dst + col0 + 4 * quad) = v;
+      continue;
+    }
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       const int c = col0 + 4 * quad + i;
@@ -606,12 +615,13 @@ extern "C" int ls_heads_product(int dtype, const void* x, long ldx, int x_stride
   LS_REQUIRE(reinterpret_cast<uintptr_t>(w) % 16 == 0, "heads_product: the weights must be 16-byte aligned");
   const int x_aligned = reinterpret_cast<uintptr_t>(x) % 16 == 0 && ldx % vec == 0 && x_stride % vec == 0 && K % vec == 0;
   hipStream_t s = reinterpret_cast<hipStream_t>(stream);
+  const int out_vec = ldo % 4 == 0 && o_stride % 4 == 0 && reinterpret_cast<uintptr_t>(out) % (dtype == kF32 ? 16 : 8) == 0;
   const bool many = n_rows > 64;
   const int rows_a_block = many ? 64 : 16;
   const dim3 grid((n_rows + rows_a_block - 1) / rows_a_block, H, (N + 63) / 64);
 #define LS_HEADS(T_, RT_)                                                                                            \
   hipLaunchKernelGGL((heads_product_kernel<T_, RT_>), grid, dim3(256), 0, s, (const T_*)x, ldx, x_stride, (const T_*)w, N, \
-                     K, n_rows, (T_*)out, ldo, o_stride, x_aligned)
+                     K, n_rows, (T_*)out, ldo, o_stride, x_aligned, out_vec)
   if (dtype == kF32) {
     if (many) LS_HEADS(float, 4); else LS_HEADS(float, 1);
   } else {

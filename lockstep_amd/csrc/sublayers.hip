@@ -209,6 +209,10 @@ __device__ __forceinline__ void channel_gates(float a, float v, float& keep, flo
   write = Gates<T>::sigmoid(a) * (v >= 0.f ? v + 0.5f : Gates<T>::sigmoid(v));
 }
 
+// A barrier between the waves' LDS writes and reads that waits for this wave's LDS operations only: the global
+// loads of the next round stay on their way across it.
+__device__ __forceinline__ void round_barrier() { __asm__ volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
+
 constexpr int kRunTokens = 8;
 constexpr int kRunCols = 16;
 constexpr int kRunWaves = 16;
@@ -277,7 +281,7 @@ __global__ __launch_bounds__(64 * kRunWaves) void channel_recurrence_kernel(
       pairs[set][wv][l16][0] = wA;
       pairs[set][wv][l16][1] = wB;
     }
-    __syncthreads();
+    round_barrier();
     float front = 0.f;
 #pragma unroll
     for (int s = 0; s < kRunWaves; ++s) {

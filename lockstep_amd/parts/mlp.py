@@ -7,6 +7,8 @@ kernel."""
 
 from __future__ import annotations
 
+import math
+
 import torch
 
 from ..config.base import PartSpec
@@ -141,8 +143,9 @@ class MLP(FeedForward):
         self.w_up = rt.matrix(weights.get(up))
         self.w_down = rt.matrix(weights.get(down))
         if self.activation == "xielu":
-            both = torch.nn.functional.softplus(weights.get(act).to(torch.float64).reshape(2), threshold=40.0)
-            self.factors = rt.vector((both + torch.tensor([0.0, 0.5], dtype=torch.float64)).to(torch.float32))
+            p, q = weights.get(act).to(torch.float64).reshape(2).tolist()
+            softplus = [max(v, 0.0) + math.log1p(math.exp(-abs(v))) for v in (p, q)]
+            self.factors = rt.vector(torch.tensor([softplus[0], 0.5 + softplus[1]], dtype=torch.float64))
 
     def forward(self, ctx, x, out, accumulate: bool, defer: bool = False):
         from .base import project_out
