@@ -41,7 +41,9 @@ design (chunked and biased attention with a sink and an output gate, routed expe
 attention, attention over a cached latent, experts named by a table) or, with ``--designs qwen3,toripel,narurax``,
 the Narurax design (an embedding that adds a table of token pairs, mixer inputs shifted towards the token before, the
 delta rule with a decay a channel, attention whose weights are mixed over the heads, attention with a norm a head,
-windows that keep the first tokens, experts with sigmoid scores on their input; ``--designs``
+windows that keep the first tokens, experts with sigmoid scores on their input) or, with ``--designs
+qwen3,toripel,tukavik``, the Tukavik design (norms on both sides of every sublayer, averages over depth, a recurrence of one
+number a channel, attention over a cached latent without positions, two-matrix feed-forwards with xIELU; ``--designs``
 chooses) beside the Qwen3 decoder at the same layer sizes (width, feed-forward, heads, head size, layers, vocabulary), both
 with random weights: prefill of one prompt and decode steps at batch 1 and 8, each with its
 fraction of the roofline.

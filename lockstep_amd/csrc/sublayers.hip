@@ -30,7 +30,7 @@ struct SeqMeta {  // one per sequence of the step (all int32), as the step's upl
 // norm(v) = (v - m) / sqrt(mean((v - m)^2) + eps) * w with m the row's mean (`centred`), or 0 without it.
 // With a row list the rows rows[r] are read and only `out` is written.
 // Thread t of 256 owns the elements 1024 c + 4 t + {0..3}, c ascending; a sum adds them in that order, then a
-// butterfly over the wave and the wave sums in wave order.  Slices and results are requested eight at a time.
+// butterfly over the wave and the wave sums in wave order.  Slices and results are requested eight at a time (fewer in wide rows).
 // ---------------------------------------------------------------------------
 constexpr int kStepWidth = 16384;  // the widest row: 16 chunks of 1024 elements stay in registers
 
@@ -100,7 +100,7 @@ __global__ __launch_bounds__(256) void residual_step_kernel(
     const float* __restrict__ post_w, float post_eps, int post_centred, float* __restrict__ results, long r_stride, int keep,
     const float* __restrict__ shares, const float* __restrict__ weight, float eps, int centred, T* __restrict__ out,
     long ld_out, const int* __restrict__ rows) {
-  constexpr int BATCH = NC <= 2 ? 8 : 4;
+  constexpr int BATCH = NC <= 2 ? 8 : NC <= 4 ? 4 : NC <= 8 ? 2 : 1;
   __shared__ float scratch[16];
   const int r_out = blockIdx.x;
   const long row = rows ? rows[r_out] : r_out;

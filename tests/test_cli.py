@@ -119,3 +119,20 @@ def test_init_writes_a_narurax_folder_from_its_preset(tmp_path):
         assert name in names, name
     assert "l1.mix.v" not in names and "l3.mlp.router" not in names and "l0.mlp.router.b" not in names and "l0.mix.a" not in names
     assert tuple(handle.shape("bigram")) == (510, 128) and tuple(handle.shape("l0.mix.dt_bias")) == (128,)
+
+
+def test_init_writes_a_tukavik_folder_from_its_preset(tmp_path):
+    from lockstep_amd.config import TukavikConfig, config_from_dir
+    from lockstep_amd.weights import SafetensorsFile
+
+    done = run("init", "--preset", "tukavik-tiny", "--out", str(tmp_path / "k"), "--seed", "2")
+    assert done.returncode == 0, done.stderr
+    config = config_from_dir(tmp_path / "k")
+    assert isinstance(config, TukavikConfig) and config.width == 128 and len(config.layers) == 4
+    handle = SafetensorsFile(tmp_path / "k" / "model.safetensors")
+    names = handle.keys()
+    for name in ("embed", "final.norm", "l0.norm1", "l0.norm1b", "l0.norm2b", "l0.mix.z.b", "l0.mix.g", "l0.mlp.act", "l0.dwa",
+                 "l1.mix.q", "l1.mix.dkv.norm", "l1.mix.uv", "l3.mix.dq.norm", "l3.mix.uq", "l3.dwa"):
+        assert name in names, name
+    assert "head" not in names and "l3.mix.dkv" not in names and "l2.mlp.up" not in names and "l1.mix.dq" not in names
+    assert tuple(handle.shape("l3.dwa")) == (5,) and tuple(handle.shape("l1.mix.dkv")) == (40, 128)
