@@ -18,7 +18,9 @@ LIB_DIR = pathlib.Path(__file__).resolve().parent.parent / "lockstep_amd" / "_li
 SMALL = 64                                              # bytes a lane that need no entry here
 MAY_SPILL = ("attention_wide_kernelIfLi8E",)          # float, row blocks of 128: 288 bytes a lane at head size 128
 MAY_SPILL_AT_HEAD_256 = ("attention_",)               # every float instance at a head size of 256, and some bfloat16
-MAY_SPILL_AT_KEYS_OVER_256 = ("sink_attention_",)     # sink attention with keys of more than 256 elements: correct, not fast
+# sink attention with keys of more than 256 or values of more than 128 elements (a library of such a shape is built when a
+# model first asks for it): correct, not fast, or the instances of four row tiles, which only measurements use
+MAY_SPILL_AT_WIDE_HEADS = ("sink_attention_",)
 
 
 def code_object_notes(blob: bytes):
@@ -69,13 +71,13 @@ def test_no_kernel_calls_a_function_and_only_known_ones_spill():
     for lib in LIBS:
         head_256 = "attention256" in lib.name
         sizes = lib.name.split("sink")[1].split("-")[0].split("x") if "sink" in lib.name else None
-        wide_keys = sizes is not None and int(sizes[0]) > 256
+        wide_heads = sizes is not None and (int(sizes[0]) > 256 or int(sizes[1]) > 128)
         for kernel in kernels_of(lib):
             seen += 1
             name = kernel[".name"]
             assert not kernel.get(".uses_dynamic_stack", False), f"{lib.name}: {name} calls a function"
             scratch = kernel.get(".private_segment_fixed_size", 0)
-            allowed = MAY_SPILL + (MAY_SPILL_AT_HEAD_256 if head_256 else ()) + (MAY_SPILL_AT_KEYS_OVER_256 if wide_keys else ())
+            allowed = MAY_SPILL + (MAY_SPILL_AT_HEAD_256 if head_256 else ()) + (MAY_SPILL_AT_WIDE_HEADS if wide_heads else ())
             if scratch > SMALL and not any(part in name for part in allowed):
                 pytest.fail(f"{lib.name}: {name} uses {scratch} bytes of scratch memory a lane")
     assert seen > 100, "the libraries' metadata was not found"
