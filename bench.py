@@ -129,8 +129,8 @@ class Workload:
                       for matrices, vectors, _, routed in self.runs)
         weights += self.head * element + self.hidden * 4                     # head and final norm
         weights += batch * self.hidden * element                             # embedding rows
-        held = sum(batch * cache_bytes(mixer.cache_spec(), context, element) for mixer in self.writers
-                   if mixer is not None)
+        held = sum(batch * cache_bytes(spec, context, element) for mixer in self.writers if mixer is not None
+                   for spec in (mixer.cache_spec(), *mixer.further_specs()))
         return weights + held
 
 

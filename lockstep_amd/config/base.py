@@ -96,13 +96,15 @@ class ScheduleEntry:
     only reads a unit that another entry fills (sharing another layer's keys
     and values).  ``state`` is a second unit, for what the layer's arrangement
     itself keeps per request between steps (``Arrangement.state_spec``), or
-    None where it keeps nothing.
+    None where it keeps nothing.  ``further``: the units of a mixer that keeps
+    more than one thing (``Mixer.further_specs``, in its order).
     """
 
     layer: int
     cache: int
     writes_cache: bool = True
     state: int | None = None
+    further: tuple[int, ...] = ()
 
 
 @dataclass(frozen=True)
@@ -127,6 +129,7 @@ class ModelSpec:
 
     def cache_units(self) -> int:
         units = [e.cache for e in self.schedule] + [e.state for e in self.schedule if e.state is not None]
+        units += [unit for e in self.schedule for unit in e.further]
         if self.embedding_state is not None:
             units.append(self.embedding_state)
         return 1 + max(units, default=-1)

@@ -4,10 +4,13 @@
 //   z[t]        = router logits of token t (float, computed by the caller's matrix product) + bias
 //   chosen(t)   = the `top` experts with the largest z[t] (the lower index wins a tie), in that order
 //   w[t, k]     = softmax over the chosen logits alone
+//                 (scoring 1: the sigmoid of each; scoring 2: the choice is made by softmax(z) + correction, within the
+//                 best groups of experts, and the weights are the chosen softmax(z) divided by their sum)
 //   expert e    : y = act(W_gate[e] x, W_up[e] x),  out = W_down[e] y
 //                 act(g, u) = g' sigmoid(alpha g') (u' + shift),  g' = min(g, limit),  u' = clamp(u, -limit, limit)
 //                 (an infinite limit, alpha 1 and shift 0: the plain gated unit silu(g) u)
 //   P[k][t]     = w[t, k] * expert chosen(t)[k] (x[t])        (float; the caller adds the slices in order)
+//                 (experts from the `real`-th on have no weights: they return x[t] itself)
 //
 // (1) route: a wave a token picks the experts and their weights.  (2) group: the (token, choice) pairs
 // are put in the order of their experts (a stable counting sort: a wave an expert counts its pairs by
@@ -37,24 +40,33 @@ constexpr int kMaxPerLane = 8;   // experts a lane holds: up to 512 experts
 
 // scoring 0: the weights are the softmax over the chosen logits; 1: each chosen expert weighs the sigmoid of its own
 // logit, and nothing is renormalised (the sigmoid grows with the logit, so the largest logits are the largest scores).
+// scoring 2: scores s = softmax over all E logits; the choice goes by s + correction, among the experts of the `keep` groups
+// (of `groups` equal runs of neighbours) whose largest choice score is largest; the weights are the chosen s divided by
+// their sum (+ kShareEps).
+constexpr float kShareEps = 1e-20f;
+
+struct Choice {
+  int scoring, groups, keep;
+  const float* correction;   // [E], scoring 2
+};
+
 __device__ __forceinline__ void pick_top(const float* __restrict__ row, const float* __restrict__ bias, int E, int top,
-                                         int lane, int* __restrict__ picked, float* __restrict__ share, int scoring) {
-  float mine[kMaxPerLane];
+                                         int lane, int* __restrict__ picked, float* __restrict__ share, const Choice& how) {
+  float mine[kMaxPerLane], score[kMaxPerLane];
 #pragma unroll
   for (int m = 0; m < kMaxPerLane; ++m) {
     const int e = lane + 64 * m;
     mine[m] = e < E ? row[e] + (bias ? bias[e] : 0.f) : 0.f;
+    score[m] = 0.f;
   }
-  unsigned taken = 0;
-  int my_pick = 0;
-  float my_value = 0.f, first = 0.f;
-  for (int k = 0; k < top; ++k) {
-    float best_v = 0.f;
-    int best = 0x7fffffff;
+  // the largest of every lane's open experts, the lower index winning a tie (0x7fffffff: none is open)
+  auto largest = [&](unsigned closed, float& best_v, int& best) LS_INLINED {
+    best_v = 0.f;
+    best = 0x7fffffff;
 #pragma unroll
     for (int m = 0; m < kMaxPerLane; ++m) {
       const int e = lane + 64 * m;
-      if (e < E && !((taken >> m) & 1u) && (best == 0x7fffffff || mine[m] > best_v)) {
+      if (e < E && !((closed >> m) & 1u) && (best == 0x7fffffff || mine[m] > best_v)) {
         best_v = mine[m];
         best = e;
       }
@@ -67,18 +79,70 @@ __device__ __forceinline__ void pick_top(const float* __restrict__ row, const fl
       best_v = take ? other_v : best_v;
       best = take ? other : best;
     }
+  };
+  unsigned taken = 0;
+  if (how.scoring == 2) {
+    float top_z;
+    int at;
+    largest(0u, top_z, at);
+    float part = 0.f;
+#pragma unroll
+    for (int m = 0; m < kMaxPerLane; ++m) {
+      score[m] = lane + 64 * m < E ? expf(mine[m] - top_z) : 0.f;
+      part = part + score[m];
+    }
+    const float inv = 1.0f / wave_sum(part);
+#pragma unroll
+    for (int m = 0; m < kMaxPerLane; ++m) {
+      score[m] = score[m] * inv;
+      if (lane + 64 * m < E) mine[m] = score[m] + how.correction[lane + 64 * m];
+    }
+    if (how.keep < how.groups) {   // the groups, best first: every pick closes its group for the next one
+      const int each = E / how.groups;
+      unsigned open = 0;
+      for (int g = 0; g < how.keep; ++g) {
+        float v;
+        int best;
+        largest(open, v, best);
+#pragma unroll
+        for (int m = 0; m < kMaxPerLane; ++m)
+          if ((lane + 64 * m) / each == best / each) open |= 1u << m;
+      }
+      taken = ~open;
+    }
+  }
+  int my_pick = 0;
+  float my_value = 0.f, first = 0.f;
+  for (int k = 0; k < top; ++k) {
+    float best_v;
+    int best;
+    largest(taken, best_v, best);
     if ((best & 63) == lane) taken |= 1u << (best >> 6);
     if (k == 0) first = best_v;
+    if (how.scoring == 2) {   // (the weight is the score without the correction)
+      float held = 0.f;
+#pragma unroll
+      for (int m = 0; m < kMaxPerLane; ++m) held = (best >> 6) == m ? score[m] : held;
+      best_v = __shfl(held, best & 63, kWave);
+    }
     if (lane == k) {
       my_pick = best;
       my_value = best_v;
     }
   }
+  if (how.scoring == 2) {
+    const float sum = wave_sum(lane < top ? my_value : 0.f);
+    if (lane < top) {
+      picked[lane] = my_pick;
+      share[lane] = my_value / (sum + kShareEps);
+    }
+    return;
+  }
   const float ex = lane < top ? expf(my_value - first) : 0.f;   // (the first pick is the largest)
   const float sum = wave_sum(ex);
   if (lane < top) {
     picked[lane] = my_pick;
-    share[lane] = scoring == 1 ? sigmoid_e(my_value) : ex / sum;
+    share[lane] = how.scoring == 1 ? sigmoid_e(my_value) : ex / sum;
   }
 }
 
@@ -95,10 +159,10 @@ __global__ __launch_bounds__(256) void route_table_kernel(const int* __restrict_
 
 __global__ __launch_bounds__(256) void route_topk_kernel(const float* __restrict__ z, long ldz,
                                                          const float* __restrict__ bias, int n_tokens, int E, int top,
-                                                         int* __restrict__ expert, float* __restrict__ weight, int scoring) {
+                                                         int* __restrict__ expert, float* __restrict__ weight, Choice how) {
   const int t = blockIdx.x * 4 + (threadIdx.x >> 6);
   if (t >= n_tokens) return;
-  pick_top(z + (long)t * ldz, bias, E, top, threadIdx.x & 63, expert + (long)t * top, weight + (long)t * top, scoring);
+  pick_top(z + (long)t * ldz, bias, E, top, threadIdx.x & 63, expert + (long)t * top, weight + (long)t * top, how);
 }
 
 // ---------------------------------------------------------------------------
@@ -183,7 +247,7 @@ __global__ __launch_bounds__(1024) void route_small_kernel(const float* __restri
                                                            float* __restrict__ weight, int* __restrict__ order,
                                                            int* __restrict__ tiles, int cap,
                                                            const int* __restrict__ token_ids, const int* __restrict__ table,
-                                                           int scoring) {
+                                                           Choice how) {
   __shared__ int picks_s[kSmallPairs];
   __shared__ float share_s[16][kMaxTop];
   __shared__ int counts_s[kSmallExperts];
@@ -198,7 +262,7 @@ __global__ __launch_bounds__(1024) void route_small_kernel(const float* __restri
     }
   }
   for (int t = w; t < n_tokens && !table; t += 16) {
-    pick_top(z + (long)t * ldz, bias, E, top, lane, picks_s + t * top, share_s[w], scoring);
+    pick_top(z + (long)t * ldz, bias, E, top, lane, picks_s + t * top, share_s[w], how);
     if (lane < top) {
       expert[(long)t * top + lane] = picks_s[t * top + lane];
       weight[(long)t * top + lane] = share_s[w][lane];
@@ -222,12 +286,13 @@ __global__ __launch_bounds__(256) void experts_gate_up_kernel(const T* __restric
                                                               const T* __restrict__ w_gate, const T* __restrict__ w_up,
                                                               int F, int K, int top, const int* __restrict__ order,
                                                               const int* __restrict__ tiles, float limit, float alpha, float shift,
-                                                              const float* __restrict__ in_weight, T* __restrict__ act, long ldy) {
+                                                              const float* __restrict__ in_weight, T* __restrict__ act, long ldy,
+                                                              int real) {
   // in_weight (or null): a pair's routing weight multiplies the expert's input, w * x, so both products are scaled
   // by it before the gated unit (the down product then adds the expert's output as it is)
   constexpr int VEC = Atom<T>::VEC, KC = Atom<T>::KCHUNK;
   const int e = tiles[4 * blockIdx.x];
-  if (e < 0) return;
+  if (e < 0 || e >= real) return;   // (an expert that returns its input has nothing to multiply)
   const int first = tiles[4 * blockIdx.x + 1], rows = tiles[4 * blockIdx.x + 2];
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
   const int l16 = lane & 15, quad = lane >> 4;
@@ -308,6 +373,19 @@ __global__ __launch_bounds__(256) void experts_gate_up_kernel(const T* __restric
   }
 }
 
+// A tile of an expert that returns its input: P[choice][token][c] = share * x[token][c] for the columns [c0, c1), the
+// routing weight multiplying the input or the output alike.
+template <typename T>
+__device__ __forceinline__ void pass_input(const T* __restrict__ x, long ldx, const float* __restrict__ share, int first, int rows,
+                                           int c0, int c1, int top, int n_tokens, int N, const int* __restrict__ order,
+                                           float* __restrict__ P) {
+  const int width = c1 - c0;
+  for (int i = threadIdx.x; i < rows * width; i += 256) {
+    const int pair = order[first + i / width], c = c0 + i % width;
+    P[((long)(pair % top) * n_tokens + pair / top) * N + c] = share[pair] * to_f32(x[(long)(pair / top) * ldx + c]);
+  }
+}
+
 // ---------------------------------------------------------------------------
 // (4) P[choice][token][:] = weight[pair] * (act[place] W_down[e]^T).  w_down [E][N][F]; P [top][n_tokens][N] float.
 // ---------------------------------------------------------------------------
@@ -316,11 +394,18 @@ __global__ __launch_bounds__(256) void experts_down_kernel(const T* __restrict__
                                                            const T* __restrict__ w_down, int N, int F, int top,
                                                            int n_tokens, const int* __restrict__ order,
                                                            const int* __restrict__ tiles,
-                                                           const float* __restrict__ weight, float* __restrict__ P) {
+                                                           const float* __restrict__ weight, float* __restrict__ P,
+                                                           const T* __restrict__ x, long ldx, const float* __restrict__ share,
+                                                           int real) {
   constexpr int VEC = Atom<T>::VEC, KC = Atom<T>::KCHUNK;
   const int e = tiles[4 * blockIdx.x];
   if (e < 0) return;
   const int first = tiles[4 * blockIdx.x + 1], rows = tiles[4 * blockIdx.x + 2];
+  if (e >= real) {   // (the whole workgroup)
+    constexpr int kCols = KS == 1 ? 64 : 16;
+    pass_input<T>(x, ldx, share, first, rows, blockIdx.y * kCols, min(N, (int)(blockIdx.y + 1) * kCols), top, n_tokens, N, order, P);
+    return;
+  }
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
   const int l16 = lane & 15, quad = lane >> 4;
   const int col0 = KS == 1 ? (blockIdx.y * 4 + w) * 16 : blockIdx.y * 16;
@@ -470,10 +555,10 @@ __global__ __launch_bounds__(256) void experts_gate_up_tiled_kernel(const T* __r
                                                                     const int* __restrict__ order,
                                                                     const int* __restrict__ tiles, float limit, float alpha,
                                                                     float shift, const float* __restrict__ in_weight,
-                                                                    T* __restrict__ act, long ldy) {
+                                                                    T* __restrict__ act, long ldy, int real) {
   __shared__ __attribute__((aligned(16))) char lds[2 * 3 * 64 * kLdsRow];
   const int e = tiles[4 * blockIdx.x];
-  if (e < 0) return;
+  if (e < 0 || e >= real) return;
   const int first = tiles[4 * blockIdx.x + 1], rows = tiles[4 * blockIdx.x + 2];
   const int col0 = blockIdx.y * 64;
   const T* a_row[2];
@@ -514,12 +599,18 @@ __global__ __launch_bounds__(256) void experts_down_tiled_kernel(const T* __rest
                                                                  const T* __restrict__ w_down, int N, int F, int top,
                                                                  int n_tokens, const int* __restrict__ order,
                                                                  const int* __restrict__ tiles,
-                                                                 const float* __restrict__ weight, float* __restrict__ P) {
+                                                                 const float* __restrict__ weight, float* __restrict__ P,
+                                                                 const T* __restrict__ x, long ldx,
+                                                                 const float* __restrict__ share, int real) {
   __shared__ __attribute__((aligned(16))) char lds[2 * 2 * 64 * kLdsRow];
   const int e = tiles[4 * blockIdx.x];
   if (e < 0) return;
   const int first = tiles[4 * blockIdx.x + 1], rows = tiles[4 * blockIdx.x + 2];
   const int col0 = blockIdx.y * 64;
+  if (e >= real) {
+    pass_input<T>(x, ldx, share, first, rows, col0, min(N, col0 + 64), top, n_tokens, N, order, P);
+    return;
+  }
   const T* a_row[2];
   const T* b_row[1][2];
 #pragma unroll
@@ -567,8 +658,12 @@ extern "C" int ls_experts_tile_capacity(int n_tokens, int E, int top, int rows_a
 // tiles [cap][4]; counts: scratch of E ints.  rows_a_tile 16, 32 or 64.
 extern "C" int ls_experts_route(const float* z, long ldz, const float* bias, int n_tokens, int E, int top,
                                 int rows_a_tile, int* expert, float* weight, int* order, int* tiles, int cap,
-                                int* counts, int scoring, void* stream) {
-  LS_REQUIRE(scoring == 0 || scoring == 1, "experts_route: scoring %d (0: softmax over the chosen, 1: sigmoid)", scoring);
+                                int* counts, int scoring, const float* correction, int groups, int keep, void* stream) {
+  LS_REQUIRE(scoring >= 0 && scoring <= 2, "experts_route: scoring %d (0: softmax over the chosen, 1: sigmoid, 2: softmax over all)",
+             scoring);
+  LS_REQUIRE(scoring != 2 || (correction && groups > 0 && keep > 0 && keep <= groups && E % groups == 0 && top <= keep * (E / groups)),
+             "experts_route: %d experts in %d groups of which %d are kept, %d a token", E, groups, keep, top);
+  const Choice how{scoring, groups, keep, correction};
   LS_REQUIRE(n_tokens > 0 && E > 0 && top > 0 && top <= E && top <= kMaxTop && ldz >= E,
              "experts_route: %d tokens, %d experts, %d chosen (at most %d)", n_tokens, E, top, kMaxTop);
   LS_REQUIRE(rows_a_tile == 16 || rows_a_tile == 32 || rows_a_tile == 64, "experts_route: tiles of %d rows", rows_a_tile);
@@ -579,10 +674,10 @@ extern "C" int ls_experts_route(const float* z, long ldz, const float* bias, int
   const int P = n_tokens * top;
   if (P <= kSmallPairs && E <= kSmallExperts) {
     hipLaunchKernelGGL(route_small_kernel, dim3(1), dim3(1024), 0, s, z, ldz, bias, n_tokens, E, top, rows_a_tile,
-                       expert, weight, order, tiles, cap, (const int*)nullptr, (const int*)nullptr, scoring);
+                       expert, weight, order, tiles, cap, (const int*)nullptr, (const int*)nullptr, how);
   } else {
     hipLaunchKernelGGL(route_topk_kernel, dim3((n_tokens + 3) / 4), dim3(256), 0, s, z, ldz, bias, n_tokens, E, top,
-                       expert, weight, scoring);
+                       expert, weight, how);
     hipLaunchKernelGGL(route_count_kernel, dim3(E), dim3(64), 0, s, expert, P, counts);
     hipLaunchKernelGGL(route_place_kernel, dim3(E), dim3(64), 0, s, expert, counts, P, E, rows_a_tile, order, tiles, cap);
   }
@@ -601,7 +696,7 @@ extern "C" int ls_experts_route_table(const int* token_ids, const int* table, in
   const int P = n_tokens * top;
   if (P <= kSmallPairs && E <= kSmallExperts) {
     hipLaunchKernelGGL(route_small_kernel, dim3(1), dim3(1024), 0, s, (const float*)nullptr, 0L, (const float*)nullptr,
-                       n_tokens, E, top, rows_a_tile, expert, weight, order, tiles, cap, token_ids, table, 0);
+                       n_tokens, E, top, rows_a_tile, expert, weight, order, tiles, cap, token_ids, table, Choice{0, 1, 1, nullptr});
   } else {
     hipLaunchKernelGGL(route_table_kernel, dim3((P + 255) / 256), dim3(256), 0, s, token_ids, table, n_tokens, top, expert,
                        weight);
@@ -617,8 +712,10 @@ extern "C" int ls_experts_apply(int dtype, const void* x, long ldx, const void* 
                                 const void* w_down, int n_tokens, int E, int top, int K, int F, int N,
                                 int rows_a_tile, const int* order, const int* tiles, int cap, const float* weight,
                                 float limit, float alpha, float shift, void* act, long ldy, float* P, int weigh_input,
-                                void* stream) {
-  // weigh_input: the routing weight multiplies the expert's input instead of its output
+                                int real, void* stream) {
+  // weigh_input: the routing weight multiplies the expert's input instead of its output.  real: experts from this one on
+  // (of the E that the tiles may name) have no weights and return their input
+  LS_REQUIRE(real > 0 && real <= E && (real == E || K == N), "experts_apply: %d of %d experts with weights", real, E);
   const float* in_weight = weigh_input ? weight : nullptr;
   const float* out_weight = weigh_input ? nullptr : weight;
   LS_REQUIRE(n_tokens > 0 && E > 0 && top > 0 && K > 0 && F > 0 && N > 0 && ldx >= K && ldy >= F, "experts_apply: bad sizes");
@@ -639,9 +736,9 @@ extern "C" int ls_experts_apply(int dtype, const void* x, long ldx, const void* 
   do {                                                                                                                \
     hipLaunchKernelGGL((experts_gate_up_kernel<T_, RT_, KS_>), grid_up, dim3(256), 0, s, (const T_*)x, ldx,           \
                        (const T_*)w_gate, (const T_*)w_up, F, K, top, order, tiles, limit, alpha, shift, in_weight,   \
-                       (T_*)act, ldy);                                                                                \
+                       (T_*)act, ldy, real);                                                                          \
     hipLaunchKernelGGL((experts_down_kernel<T_, RT_, KS_>), grid_down, dim3(256), 0, s, (const T_*)act, ldy,          \
-                       (const T_*)w_down, N, F, top, n_tokens, order, tiles, out_weight, P);                          \
+                       (const T_*)w_down, N, F, top, n_tokens, order, tiles, out_weight, P, (const T_*)x, ldx, weight, real); \
   } while (0)
   // tiles of 64 rows go through LDS where every row of every operand starts on a 16-byte boundary
   const bool staged = rows_a_tile == 64 && K % vec == 0 && F % vec == 0 && ldx % vec == 0 && ldy % vec == 0;
@@ -649,9 +746,9 @@ extern "C" int ls_experts_apply(int dtype, const void* x, long ldx, const void* 
   do {                                                                                                                \
     hipLaunchKernelGGL(experts_gate_up_tiled_kernel<T_>, grid_up, dim3(256), 0, s, (const T_*)x, ldx,                 \
                        (const T_*)w_gate, (const T_*)w_up, F, K, top, order, tiles, limit, alpha, shift, in_weight,   \
-                       (T_*)act, ldy);                                                                                \
+                       (T_*)act, ldy, real);                                                                          \
     hipLaunchKernelGGL(experts_down_tiled_kernel<T_>, grid_down, dim3(256), 0, s, (const T_*)act, ldy,                \
-                       (const T_*)w_down, N, F, top, n_tokens, order, tiles, out_weight, P);                          \
+                       (const T_*)w_down, N, F, top, n_tokens, order, tiles, out_weight, P, (const T_*)x, ldx, weight, real); \
   } while (0)
 #define LS_EXPERTS_BY_ROWS(T_)                 \
   switch (rows_a_tile) {                       \

@@ -42,7 +42,8 @@ __device__ __forceinline__ float block_sum4(float v, float* scratch) {
 //   write:  y = P[0][row] + P[1][row] + ... (slices ascending, from +0: the sublayer's output, left as slice sums);
 //           X'_t = sum_s mix[s][t] X_s + gain[t] y      for all t at once from the old copies
 //   read:   u = sum_t take[t] X'_t   (take == null: the plain sum of the copies)
-//           out = u / sqrt(mean(u^2) + eps) * weight     (T)
+//           out = (u - m) / sqrt(mean((u - m)^2) + eps) * weight + bias     (T; m the row's mean if `centred`, else 0; bias
+//           may be null)
 // Thread t of 256 owns the elements 1024 c + 4 t + {0..3}, c ascending; the sum of squares adds them in that order, then
 // a butterfly over the wave and the wave sums in wave order.  `row` = rows[r] when a row list is given.
 // ---------------------------------------------------------------------------
@@ -65,9 +66,9 @@ __global__ __launch_bounds__(256) void streams_step_kernel(float* __restrict__ X
                                                            const float* __restrict__ P, int slices, long p_stride,
                                                            const float* __restrict__ mix, const float* __restrict__ gain,
                                                            const float* __restrict__ take, const float* __restrict__ weight,
-                                                           float eps, T* __restrict__ out, long ld_out,
-                                                           const int* __restrict__ rows) {
-  __shared__ float mix_s[N * N], gain_s[N], take_s[N], scratch[4];
+                                                           const float* __restrict__ bias, int centred, float eps,
+                                                           T* __restrict__ out, long ld_out, const int* __restrict__ rows) {
+  __shared__ float mix_s[N * N], gain_s[N], take_s[N], scratch[4], sums_s[4];
   const int r_out = blockIdx.x;
   const long row = rows ? rows[r_out] : r_out;
   if (threadIdx.x < N * N) mix_s[threadIdx.x] = P ? mix[threadIdx.x] : 0.f;
@@ -123,22 +124,39 @@ __global__ __launch_bounds__(256) void streams_step_kernel(float* __restrict__ X
     for (int t = 0; t < N; ++t) sum = sum + take_s[t] * copy[t];
     if (out) *reinterpret_cast<f32x4*>(u_s + e) = sum;
 #pragma unroll
-    for (int i = 0; i < 4; ++i) part = part + sum[i] * sum[i];   // (elements beyond W are zeros)
+    for (int i = 0; i < 4; ++i) part = part + (centred ? sum[i] : sum[i] * sum[i]);   // (elements beyond W are zeros)
   }
   if (!out) return;
+  float mean = 0.f;
+  if (centred) {   // (the same for the whole launch)
+    mean = block_sum4(part, sums_s) / (float)W;
+    part = 0.f;
+#pragma unroll 1
+    for (int e = 4 * (int)threadIdx.x; e < W; e += 1024) {
+      const f32x4 u = *reinterpret_cast<const f32x4*>(u_s + e);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const float d = e + i < W ? u[i] - mean : 0.f;
+        part = part + d * d;
+      }
+    }
+  }
   const float scale = 1.0f / sqrtf(block_sum4(part, scratch) / (float)W + eps);
 #pragma unroll 1
   for (int e0 = 4 * (int)threadIdx.x; e0 < W; e0 += 1024) {
     const f32x4 u = *reinterpret_cast<const f32x4*>(u_s + e0);
     if (vec_ok) {
       const f32x4 w = *reinterpret_cast<const f32x4*>(weight + e0);
+      f32x4 b = {0.f, 0.f, 0.f, 0.f};
+      if (bias) b = *reinterpret_cast<const f32x4*>(bias + e0);
       T* dst = out + (long)r_out * ld_out + e0;
 #pragma unroll
-      for (int i = 0; i < 4; ++i) dst[i] = from_f32<T>((u[i] * scale) * w[i]);
+      for (int i = 0; i < 4; ++i) dst[i] = from_f32<T>(((u[i] - mean) * scale) * w[i] + b[i]);
     } else {
 #pragma unroll
       for (int i = 0; i < 4; ++i)
-        if (e0 + i < W) out[(long)r_out * ld_out + e0 + i] = from_f32<T>((u[i] * scale) * weight[e0 + i]);
+        if (e0 + i < W)
+          out[(long)r_out * ld_out + e0 + i] = from_f32<T>(((u[i] - mean) * scale) * weight[e0 + i] + (bias ? bias[e0 + i] : 0.f));
     }
   }
 }
@@ -522,8 +540,8 @@ extern "C" int ls_streams_max() { return kMaxStreams; }
 extern "C" int ls_streams_max_width() { return 1024 * kStreamChunks; }
 
 extern "C" int ls_streams_step(int dtype, float* X, long ldx, int n, int width, const float* P, int slices, int p_rows,
-                               const float* mix, const float* gain, const float* take, const float* weight, float eps,
-                               void* out, long ld_out, const int* rows, int n_rows, void* stream) {
+                               const float* mix, const float* gain, const float* take, const float* weight, const float* bias,
+                               int centred, float eps, void* out, long ld_out, const int* rows, int n_rows, void* stream) {
   LS_REQUIRE(n_rows > 0 && n > 0 && n <= kMaxStreams && width > 0 && width <= 1024 * kStreamChunks && ldx >= (long)n * width,
              "streams_step: %d copies of %d elements (at most %d of %d)", n, width, kMaxStreams, 1024 * kStreamChunks);
   LS_REQUIRE(X && (P || out), "streams_step: nothing to do");
@@ -537,10 +555,10 @@ extern "C" int ls_streams_step(int dtype, float* X, long ldx, int n, int width, 
   case N_:                                                                                                           \
     if (dtype == kF32)                                                                                               \
       hipLaunchKernelGGL((streams_step_kernel<float, N_>), dim3(n_rows), dim3(256), lds, s, X, ldx, width, P, slices, \
-                         p_stride, mix, gain, take, weight, eps, (float*)out, ld_out, rows);                         \
+                         p_stride, mix, gain, take, weight, bias, centred, eps, (float*)out, ld_out, rows);                         \
     else                                                                                                             \
       hipLaunchKernelGGL((streams_step_kernel<bf16_t, N_>), dim3(n_rows), dim3(256), lds, s, X, ldx, width, P, slices, \
-                         p_stride, mix, gain, take, weight, eps, (bf16_t*)out, ld_out, rows);                        \
+                         p_stride, mix, gain, take, weight, bias, centred, eps, (bf16_t*)out, ld_out, rows);                        \
     break;
   switch (n) {
     LS_STREAMS(1) LS_STREAMS(2) LS_STREAMS(3) LS_STREAMS(4) LS_STREAMS(5) LS_STREAMS(6) LS_STREAMS(7) LS_STREAMS(8)

@@ -158,7 +158,7 @@ __global__ __launch_bounds__(256) void talk_qkv_kernel(
 // Post pass of an attention projection raw [T][ld] float = q (H heads of D) | k (G of D) | v (G of DV, absent
 // when the keys are the values) | whatever follows (an output gate, which this pass leaves alone):
 //   biases added (bias [H*D + G*D (+ G*DV)] or null);
-//   v = k as projected, with its bias, before any norm (keys_are_values; DV == D);
+//   v = k as projected, with its bias, before any norm (keys_are_values; DV == D); values are stored times v_scale;
 //   q and k each divided by the root mean square over ALL their heads at once (the whole projection is one
 //   vector: x / sqrt(mean(x^2) + eps)), times a weight an element (q_norm [H*D], k_norm [G*D]; null: no norm);
 //   or, with per_head, every head of q and of k divided by its own root mean square over D (per_head 1: no weights;
@@ -189,7 +189,7 @@ __global__ __launch_bounds__(256) void qkv_post_kernel(
     const float* __restrict__ cos_table, const float* __restrict__ sin_table, int rot, int neighbours,
     const int* __restrict__ tok_seq, const int* __restrict__ tok_pos, const SeqMeta* __restrict__ seqs,
     const int* __restrict__ table, int table_stride, T* __restrict__ q_out, long ldq, T* __restrict__ k_pages,
-    T* __restrict__ v_pages, int page_size) {
+    T* __restrict__ v_pages, int page_size, float v_scale) {
   __shared__ float scratch[4];
   __shared__ float head_scale[kMaxNormedHeads];
   const int t = blockIdx.x;
@@ -277,7 +277,7 @@ __global__ __launch_bounds__(256) void qkv_post_kernel(
     } else {
       const int c = e - oq - ok;
       const int from = keys_are_values ? nq + c : nq + nk + c;
-      const float v = row[from] + (bias ? bias[from] : 0.f);
+      const float v = (row[from] + (bias ? bias[from] : 0.f)) * v_scale;
       const int g = c / DV, i = c % DV;
       v_pages[(((long)page * G + g) * DV + i) * page_size + slot] = from_f32<T>(v);
     }
@@ -504,25 +504,32 @@ __global__ __launch_bounds__(1024) void linrec_kernel(const float* __restrict__ 
 
 // ---------------------------------------------------------------------------
 // Per (token, head): x [DV] float divided by its root mean square (eps inside the root), times
-// weight[c] if given, times silu (gate_act 0) or sigmoid (gate_act 1) of gate[t][head * DV + c] if given; stored as T.  One wave a
+// weight[c] (weight_each 0) or weight[head * weight_each + c] if given, times silu (gate_act 0) or sigmoid (gate_act 1) of gate[t][head * DV + c] if given; stored as T.  One wave a
 // head: lane i adds the squares of the elements i, i + 64, ... ascending, then a butterfly.
+// With `denom` [T][H][4] (floor, read-out in the last two places) the head is first divided by max(|read-out|, floor) +
+// denom_eps.
 // ---------------------------------------------------------------------------
 template <typename T>
 __global__ __launch_bounds__(256) void head_norm_gate_kernel(const float* __restrict__ x, long ldx, int n_tokens,
-                                                             int H, int DV, const float* __restrict__ weight,
+                                                             int H, int DV, const float* __restrict__ weight, int weight_each,
                                                              const float* __restrict__ gate, long ldg, int gate_act,
+                                                             const float* __restrict__ denom, float denom_eps,
                                                              float eps, T* __restrict__ out, long ldo) {
   const long unit = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
   if (unit >= (long)n_tokens * H) return;
   const int t = (int)(unit / H), head = (int)(unit % H), lane = threadIdx.x & 63;
   const float* src = x + (long)t * ldx + head * DV;
+  const float share = denom ? 1.0f / (fmaxf(fabsf(denom[4 * unit + 3]), denom[4 * unit + 2]) + denom_eps) : 1.0f;
   float part = 0.f;
-  for (int c = lane; c < DV; c += 64) part = part + src[c] * src[c];
+  for (int c = lane; c < DV; c += 64) {
+    const float v = denom ? src[c] * share : src[c];
+    part = part + v * v;
+  }
   const float total = wave_sum(part);
   const float scale = 1.0f / sqrtf(total / (float)DV + eps);
   for (int c = lane; c < DV; c += 64) {
-    float v = src[c] * scale;
-    if (weight) v = v * weight[c];
+    float v = (denom ? src[c] * share : src[c]) * scale;
+    if (weight) v = v * weight[(long)head * weight_each + c];
     if (gate) {
       const float z = gate[(long)t * ldg + head * DV + c];
       v = v * (gate_act == 1 ? sigmoidf_(z) : siluf_(z));
@@ -804,7 +811,7 @@ extern "C" int ls_qkv_post(int dtype, const float* raw, long ld, int n_tokens, i
                            const float* cos_table, const float* sin_table, int rot, int neighbours,
                            int table_positions, int max_pos, const int* tok_seq, const int* tok_pos, const void* seqs,
                            const int* table, int table_stride, void* q_out, long ldq, void* k_pages, void* v_pages,
-                           int page_size, void* stream) {
+                           int page_size, float v_scale, void* stream) {
   LS_REQUIRE(n_tokens > 0 && H > 0 && G > 0 && D > 0 && Dp >= D && DV > 0 && H % G == 0, "qkv_post: bad head sizes");
   LS_REQUIRE(!keys_are_values || DV == D, "qkv_post: keys of %d elements cannot be values of %d", D, DV);
   const long width = (long)H * D + (long)G * D + (keys_are_values ? 0 : (long)G * DV);
@@ -827,7 +834,7 @@ extern "C" int ls_qkv_post(int dtype, const float* raw, long ld, int n_tokens, i
 #define LS_QKV_POST(T_)                                                                                               \
   hipLaunchKernelGGL(qkv_post_kernel<T_>, dim3(n_tokens, pieces), dim3(256), 0, s, raw, ld, H, G, D, Dp, DV, keys_are_values, per_head, \
                      bias, q_norm, k_norm, eps, cos_table, sin_table, rot, neighbours, tok_seq, tok_pos,              \
-                     (const SeqMeta*)seqs, table, table_stride, (T_*)q_out, ldq, (T_*)k_pages, (T_*)v_pages, page_size)
+                     (const SeqMeta*)seqs, table, table_stride, (T_*)q_out, ldq, (T_*)k_pages, (T_*)v_pages, page_size, v_scale)
   if (dtype == kF32)
     LS_QKV_POST(float);
   else if (dtype == kBF16)
@@ -886,19 +893,19 @@ extern "C" int ls_linrec(int mode, const float* raw, long ld, int q_at, int ab_a
 }
 
 extern "C" int ls_head_norm_gate(int out_dtype, const float* x, long ldx, int n_tokens, int H, int DV,
-                                 const float* weight, const float* gate, long ldg, int gate_act, float eps, void* out,
-                                 long ldo, void* stream) {
+                                 const float* weight, int weight_each, const float* gate, long ldg, int gate_act,
+                                 const float* denom, float denom_eps, float eps, void* out, long ldo, void* stream) {
   LS_REQUIRE(n_tokens > 0 && H > 0 && DV > 0 && x && out && ldx >= (long)H * DV && ldo >= (long)H * DV &&
-                 (!gate || ldg >= (long)H * DV) && (gate_act == 0 || gate_act == 1),
+                 (!gate || ldg >= (long)H * DV) && (gate_act == 0 || gate_act == 1) && (weight_each == 0 || weight_each == DV),
              "head_norm_gate: bad sizes");
   hipStream_t s = reinterpret_cast<hipStream_t>(stream);
   dim3 grid((unsigned)(((long)n_tokens * H + 3) / 4));
   if (out_dtype == kF32)
-    hipLaunchKernelGGL(head_norm_gate_kernel<float>, grid, dim3(256), 0, s, x, ldx, n_tokens, H, DV, weight, gate, ldg,
-                       gate_act, eps, (float*)out, ldo);
+    hipLaunchKernelGGL(head_norm_gate_kernel<float>, grid, dim3(256), 0, s, x, ldx, n_tokens, H, DV, weight,
+                       weight_each, gate, ldg, gate_act, denom, denom_eps, eps, (float*)out, ldo);
   else if (out_dtype == kBF16)
-    hipLaunchKernelGGL(head_norm_gate_kernel<bf16_t>, grid, dim3(256), 0, s, x, ldx, n_tokens, H, DV, weight, gate,
-                       ldg, gate_act, eps, (bf16_t*)out, ldo);
+    hipLaunchKernelGGL(head_norm_gate_kernel<bf16_t>, grid, dim3(256), 0, s, x, ldx, n_tokens, H, DV, weight,
+                       weight_each, gate, ldg, gate_act, denom, denom_eps, eps, (bf16_t*)out, ldo);
   else
     return fail("head_norm_gate: unknown dtype %d", out_dtype);
   return check_launch("head_norm_gate");

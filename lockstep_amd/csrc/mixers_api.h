@@ -39,7 +39,7 @@ int ls_qkv_post(int dtype, const float* raw, long ld, int n_tokens, int H, int G
                 int per_head, const float* bias, const float* q_norm, const float* k_norm, float eps, const float* cos_table,
                 const float* sin_table, int rot, int neighbours, int table_positions, int max_pos, const int* tok_seq,
                 const int* tok_pos, const void* seqs, const int* table, int table_stride, void* q_out, long ldq,
-                void* k_pages, void* v_pages, int page_size, void* stream);
+                void* k_pages, void* v_pages, int page_size, float v_scale, void* stream);
 
 // Linear recurrence S_t = diag(a_t) S_(t-1) + b_t v_t^T, o_t = S_t^T q_t over the tokens of every request of the
 // step, state [slots][H][D][DV] float (mode 0: HGRN2 gates from p0 = lower bounds [H*D] and p1 = gate bias or null;
@@ -53,9 +53,11 @@ int ls_linrec(int mode, const float* raw, long ld, int q_at, int ab_at, int v_at
               float* gates, float* out, long ldo, void* stream);
 
 // Per (token, head): x [DV] / sqrt(mean(x^2) + eps), times weight [DV] and silu(gate) (gate_act 0) or sigmoid(gate)
-// (gate_act 1) where given.
+// (gate_act 1) where given.  weight_each 0: one weight vector for all heads; DV: one a head.  denom [T][H][4] (or null):
+// the head is divided by max(|denom[3]|, denom[2]) + denom_eps first.
 int ls_head_norm_gate(int out_dtype, const float* x, long ldx, int n_tokens, int H, int DV, const float* weight,
-                      const float* gate, long ldg, int gate_act, float eps, void* out, long ldo, void* stream);
+                      int weight_each, const float* gate, long ldg, int gate_act, const float* denom, float denom_eps,
+                      float eps, void* out, long ldo, void* stream);
 
 // out [T][ld_out] float = table[token] * scale + pairs[(token before * mul_prev + token * mul_cur) mod buckets]; row
 // `buckets` of pairs for a request's first token.  state: one int a slot, the last token of the request so far.
@@ -76,12 +78,13 @@ int ls_token_shift(int out_dtype, const float* n, long ldn, const float* mu, con
 
 // A residual stream of n copies X [rows][n][width] float.  Write (P given): y = P[0][row] + P[1][row] + ..., then
 // X'_t = sum_s mix[s][t] X_s + gain[t] y for all copies at once.  Read (out given): u = sum_t take[t] X'_t (take null:
-// the plain sum), out [n_rows][ld_out] = u / sqrt(mean(u^2) + eps) * weight.  rows: the rows to take, or null.
+// the plain sum), out [n_rows][ld_out] = (u - m) / sqrt(mean((u - m)^2) + eps) * weight + bias (m the mean if
+// `centred`, else 0; bias may be null).  rows: the rows to take, or null.
 int ls_streams_max();
 int ls_streams_max_width();
 int ls_streams_step(int dtype, float* X, long ldx, int n, int width, const float* P, int slices, int p_rows,
-                    const float* mix, const float* gain, const float* take, const float* weight, float eps, void* out,
-                    long ld_out, const int* rows, int n_rows, void* stream);
+                    const float* mix, const float* gain, const float* take, const float* weight, const float* bias, int centred,
+                    float eps, void* out, long ld_out, const int* rows, int n_rows, void* stream);
 
 // Post pass of the down projections of attention over a latent, raw = a (QR) | c (CR) | r (RD): a and c normalised
 // with their weights, r rotated in neighbouring pairs; a -> a_out, c | r -> key pages (heads of Dp elements, one
@@ -118,12 +121,12 @@ int ls_delta_rule(const float* raw, long ld, int n_tokens, int G, int H, int D, 
 
 // Between two sublayers of a residual stream X [.][width] float (see sublayers.hip): y = P[0][row] + P[1][row] + ...;
 // x = X[row] + norm(y) (post_w null: + y); results[keep][row] = x (results [.][r_rows][width] or null); x = the sum of
-// shares[j] results[j][row] over j = 0 .. keep (shares null: x); X[row] = x; out = norm(x).  A norm subtracts the row's
+// shares[j] results[j][row] over j = 0 .. keep (shares null: x); X[row] = x; out = norm(x) + bias (or null).  A norm subtracts the row's
 // mean when `centred`.  rows: the rows to read, or null for the first n_rows; with it only out is written.
 int ls_residual_step_max_width();
 int ls_residual_step(int dtype, float* X, long ldx, int width, const float* P, int slices, int p_rows, const float* post_w,
                      float post_eps, int post_centred, float* results, int r_rows, int keep, const float* shares,
-                     const float* weight, float eps, int centred, void* out, long ld_out, const int* rows, int n_rows,
+                     const float* weight, const float* bias, float eps, int centred, void* out, long ld_out, const int* rows, int n_rows,
                      void* stream);
 
 // One number a channel: S_t = (1 - z) S_(t-1) + z c with z = sigmoid(a + a_b), c = v + 1/2 where v = u + u_b >= 0, else
@@ -136,6 +139,43 @@ int ls_channel_recurrence(int dtype, const float* raw, long ld, int a_at, int u_
 // out [T][ld_out] float = table[token] * scale + (sin(p freq[i]), cos(p freq[i])) at the elements (2i, 2i + 1).
 int ls_embed_positions(int dtype, const int* tokens, const int* tok_pos, const void* table, int vocab, const double* freq,
                        float* out, int n_tokens, int width, long ld_out, float scale, void* stream);
+
+// Matrix memories with one gate a head and token (see memory.hip): S_t = a S_(t-1) + b k v^T, o = S^T q (+ skip v).  The
+// rows of head h of token t stand at p + t * ld + (h / share) * each; gates [T][H][4] float hold (log a, b, floor, n . q);
+// state [slots][state_stride] float starts with S [H][N][DV], and with `norm` n [H][N] behind it; out [T][ldo] float.
+int ls_memory_max_rows();
+int ls_memory_chunk();
+// A convolution a channel with silu over x | B | C of raw -> conv [T][C], and the gates from dt; ring [M][C] of the last
+// inputs at ring_at in the state (position p in row p mod M).  taps [M][C].
+int ls_conv_gates(const float* raw, long ld, int x_at, int dt_at, int n_tokens, int C, int H, int M, const float* taps,
+                  const float* bias, const float* a_log, const float* dt_bias, const int* tok_seq, const int* tok_pos,
+                  const void* seqs, int n_seqs, float* state, long state_stride, long ring_at, float* conv, float* gates,
+                  void* stream);
+// Exponential gates with a running maximum, kept as two numbers a head at m_at in the state.
+int ls_exp_gates(const float* raw, long ld, int i_at, int f_at, int H, const float* i_bias, const float* f_bias, float cap,
+                 const void* seqs, int n_seqs, float* state, long state_stride, long m_at, float* gates, void* stream);
+// Token by token, for the requests of at most `longest` tokens.
+int ls_memory_walk(const float* q, long ldq, int q_each, int q_share, const float* k, long ldk, int k_each, int k_share,
+                   const float* v, long ldv, int v_each, float* gates, int H, int N, int DV, float q_scale, const float* skip,
+                   int norm, const void* seqs, int n_seqs, int longest, float* state, long state_stride, float* out, long ldo,
+                   void* stream);
+// Chunks of 64 tokens: items [n_items][2] (request of the step, chunk), runs [n_runs][4] (request, first item, items, 0);
+// scratch states [n_items][E] with E = H N DV (+ H N), decays [n_items][H].
+int ls_memory_chunks(const float* q, long ldq, int q_each, int q_share, const float* k, long ldk, int k_each, int k_share,
+                     const float* v, long ldv, int v_each, float* gates, int H, int N, int DV, float q_scale, const float* skip,
+                     int norm, const void* seqs, const int* items, int n_items, const int* runs, int n_runs, float* states, long E,
+                     float* decays, float* state, long state_stride, float* out, long ldo, void* stream);
+// A step of single tokens in one launch: convolution and gates (space_token) or exponential gates (exp_token), the update
+// and the read.
+int ls_space_token(const float* raw, long ld, int x_at, int dt_at, int C, int G, int M, long ring_at, const float* taps,
+                   const float* conv_bias, const float* a_log, const float* dt_bias, const float* skip, int H, int N, int DV,
+                   const void* seqs, int n_seqs, float* state, long state_stride, float* out, long ldo, void* stream);
+int ls_exp_token(const float* raw, long ld, int q_at, int k_at, int v_at, int i_at, int f_at, long m_at, const float* i_bias,
+                 const float* f_bias, float cap, float q_scale, int H, int N, int DV, const void* seqs, int n_seqs, float* state,
+                 long state_stride, float* gates, float* out, long ldo, void* stream);
+// y * silu(z), divided by its root mean square in each of `parts` equal runs, times weight [inner].
+int ls_gated_parts_norm(int out_dtype, const float* y, long ldy, const float* z, long ldz, int n_tokens, int inner, int parts,
+                        const float* weight, float eps, void* out, long ldo, void* stream);
 
 int ls_listed_index(const char* name);
 int ls_call_listed(int index, const long long* words, int n);

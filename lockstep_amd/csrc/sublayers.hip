@@ -27,7 +27,7 @@ struct SeqMeta {  // one per sequence of the step (all int32), as the step's upl
 //   x = shares[0] results[0][row] + ... + shares[keep] x      (shares null: x stays)
 //   X[row] = x
 //   out = norm(x)                          (T; out null: nothing)
-// norm(v) = (v - m) / sqrt(mean((v - m)^2) + eps) * w with m the row's mean (`centred`), or 0 without it.
+// norm(v) = (v - m) / sqrt(mean((v - m)^2) + eps) * w (+ bias, for the last of the two; it may be null) with m the row's mean (`centred`), or 0 without it.
 // With a row list the rows rows[r] are read and only `out` is written.
 // Thread t of 256 owns the elements 1024 c + 4 t + {0..3}, c ascending; a sum adds them in that order, then a
 // butterfly over the wave and the wave sums in wave order.  Slices and results are requested eight at a time (fewer in wide rows).
@@ -98,8 +98,8 @@ template <typename T, int NC, bool VEC>
 __global__ __launch_bounds__(256) void residual_step_kernel(
     float* __restrict__ X, long ldx, int W, const float* __restrict__ P, int slices, long p_stride,
     const float* __restrict__ post_w, float post_eps, int post_centred, float* __restrict__ results, long r_stride, int keep,
-    const float* __restrict__ shares, const float* __restrict__ weight, float eps, int centred, T* __restrict__ out,
-    long ld_out, const int* __restrict__ rows) {
+    const float* __restrict__ shares, const float* __restrict__ weight, const float* __restrict__ bias, float eps, int centred,
+    T* __restrict__ out, long ld_out, const int* __restrict__ rows) {
   constexpr int BATCH = NC <= 2 ? 8 : NC <= 4 ? 4 : NC <= 8 ? 2 : 1;
   __shared__ float scratch[16];
   const int r_out = blockIdx.x;
@@ -171,6 +171,10 @@ __global__ __launch_bounds__(256) void residual_step_kernel(
 #pragma unroll
   for (int c = 0; c < NC; ++c) w[c] = step_load<VEC>(weight, 1024 * c + e0, W);
   step_norm<NC>(x, w, W, eps, centred, scratch + 8);
+  if (bias) {
+#pragma unroll
+    for (int c = 0; c < NC; ++c) x[c] = x[c] + step_load<VEC>(bias, 1024 * c + e0, W);
+  }
   T* dst = out + (long)r_out * ld_out;
 #pragma unroll
   for (int c = 0; c < NC; ++c) {
@@ -354,7 +358,7 @@ extern "C" int ls_residual_step_max_width() { return kStepWidth; }
 
 extern "C" int ls_residual_step(int dtype, float* X, long ldx, int width, const float* P, int slices, int p_rows,
                                 const float* post_w, float post_eps, int post_centred, float* results, int r_rows, int keep,
-                                const float* shares, const float* weight, float eps, int centred, void* out, long ld_out,
+                                const float* shares, const float* weight, const float* bias, float eps, int centred, void* out, long ld_out,
                                 const int* rows, int n_rows, void* stream) {
   LS_REQUIRE(n_rows > 0 && width > 0 && width <= kStepWidth && ldx >= width && X, "residual_step: rows of %d elements (at most %d)",
              width, kStepWidth);
@@ -369,11 +373,11 @@ extern "C" int ls_residual_step(int dtype, float* X, long ldx, int width, const 
   hipStream_t s = reinterpret_cast<hipStream_t>(stream);
   auto aligned = [](const void* p) { return reinterpret_cast<uintptr_t>(p) % 16 == 0; };
   const bool vec = width % 4 == 0 && ldx % 4 == 0 && aligned(X) && aligned(P) && aligned(post_w) && aligned(results) &&
-                   aligned(weight);
+                   aligned(weight) && aligned(bias);
   const long p_stride = (long)p_rows * width, r_stride = (long)r_rows * width;
 #define LS_STEP(T_, NC_, VEC_)                                                                                          \
   hipLaunchKernelGGL((residual_step_kernel<T_, NC_, VEC_>), dim3(n_rows), dim3(256), 0, s, X, ldx, width, P, slices,    \
-                     p_stride, post_w, post_eps, post_centred, results, r_stride, keep, shares, weight, eps, centred,   \
+                     p_stride, post_w, post_eps, post_centred, results, r_stride, keep, shares, weight, bias, eps, centred, \
                      (T_*)out, ld_out, rows)
 #define LS_STEP_VEC(T_, NC_) \
   if (vec) LS_STEP(T_, NC_, true); else LS_STEP(T_, NC_, false)

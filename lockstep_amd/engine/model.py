@@ -67,6 +67,9 @@ class Model:
                 raise ValueError(f"the schedule names layer {run.layer}, the model has {len(self.layers)}")
             if (run.state is None) != (self.layers[run.layer].state_spec() is None):
                 raise ValueError(f"layer {run.layer} keeps state of its own exactly when its schedule entry names a unit for it")
+            mixer = self.layers[run.layer].mixer
+            if len(run.further) != (0 if mixer is None else len(mixer.further_specs())):
+                raise ValueError(f"the schedule names {len(run.further)} further cache units for layer {run.layer}")
         # an embedding that keeps something per request (the token before) finds its unit here
         embedding_spec = self.embedding.state_spec() if hasattr(self.embedding, "state_spec") else None
         if (self.spec.embedding_state is None) != (embedding_spec is None):
@@ -137,6 +140,8 @@ class Model:
             mixer = self.layers[run.layer].mixer
             if run.writes_cache and mixer is not None:
                 units[run.cache] = mixer.cache_spec()
+                for unit, spec in zip(run.further, mixer.further_specs()):
+                    units[unit] = spec
             if run.state is not None:
                 units[run.state] = self.layers[run.layer].state_spec()
         if self.spec.embedding_state is not None:

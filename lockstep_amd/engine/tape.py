@@ -95,6 +95,9 @@ class RunKinds:
             if getattr(run, "state", None) is not None:
                 for i, t in enumerate(cache.unit_tensors(run.state)):
                     tensors[f"state[{i}]"] = t
+            for u, unit in enumerate(getattr(run, "further", ())):
+                for i, t in enumerate(cache.unit_tensors(unit)):
+                    tensors[f"further[{u}][{i}]"] = t
             group = cache.unit_place.get(run.cache, (None,))[0]
             self.addresses.append({name: (t.data_ptr(), t.numel() * t.element_size()) for name, t in tensors.items()})
             if not repeatable_tree(layer):

@@ -13,6 +13,7 @@ Two kinds of library exist:
                     over a latent, a product a head, the gated delta rule; the step
                     between sublayers that are normalised on both sides, with an average
                     over depth, a recurrence of one number a channel, position vectors;
+                    matrix memories with one gate a head (state space, exponential gates);
 ``talking<shape>``  attention whose heads' scores are mixed before the softmax,
                     for one shape (query heads, kv heads, key and value size).
 ``sink<D>x<DV>``    grouped-query attention with a sink in the softmax, windows or
@@ -52,7 +53,7 @@ FLAGS = [
 ]
 CORE_SOURCES = ("core.hip", "gemm.hip", "sample.hip")
 ATTENTION_SOURCES = ("attention.hip",)
-MIXERS_SOURCES = ("mixers.hip", "latent_delta.hip", "sublayers.hip")
+MIXERS_SOURCES = ("mixers.hip", "latent_delta.hip", "sublayers.hip", "memory.hip")
 TALKING_SOURCES = ("talking_attention.hip",)
 SINK_SOURCES = ("sink_attention.hip",)
 EXPERTS_SOURCES = ("experts.hip",)

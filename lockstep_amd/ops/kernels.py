@@ -937,17 +937,23 @@ class Kernels:
             _ptr(out), c_long(out.stride(0)), _stream()))
 
     def head_norm_gate(self, x: torch.Tensor, heads: int, vdim: int, weight, gate, eps: float, out: torch.Tensor,
-                       gate_act: str = "silu") -> None:
+                       gate_act: str = "silu", denom=None, denom_eps: float = 0.0) -> None:
         """Per (token, head): ``x / sqrt(mean(x^2) + eps)`` over the head's ``vdim`` values, times ``weight
         [vdim]`` and ``silu(gate)`` or, with ``gate_act = "sigmoid"``, ``sigmoid(gate)`` (float32 rows like ``x``)
-        where given; ``x`` float32 ``[T, heads*vdim]``."""
+        where given; ``x`` float32 ``[T, heads*vdim]``.  A weight of ``heads*vdim`` elements is one vector a head.  ``denom``
+        (float32 ``[T, heads, 4]``, its last two places a floor and a read-out): every head is first divided by ``max(|read-out|,
+        floor) + denom_eps``."""
         if gate_act not in ("silu", "sigmoid"):
             raise KernelError(f"head_norm_gate: the gate's activation is silu or sigmoid, got {gate_act!r}")
         _rows_ok(x, "head_norm_gate x"); _rows_ok(out, "head_norm_gate out")
         if not (x.dtype == torch.float32 and x.shape[1] == heads * vdim and out.shape == x.shape and out.dtype in DTYPE_CODE):
             raise KernelError("head_norm_gate reads float32 [T, heads*vdim] and writes the same shape")
+        each = 0
         if weight is not None:
-            self._f32_vector(weight, vdim, "head_norm_gate weight")
+            each = vdim if weight.numel() == heads * vdim else 0
+            self._f32_vector(weight, heads * vdim if each else vdim, "head_norm_gate weight")
+        if denom is not None:
+            self._f32_vector(denom, x.shape[0] * heads * 4, "head_norm_gate denom")
         ldg = 0
         if gate is not None:
             if not (gate.is_cuda and gate.dtype == torch.float32 and gate.dim() == 2 and gate.stride(1) == 1
@@ -959,7 +965,8 @@ class Kernels:
         lib = self.mixers_lib()
         self._launch(lib, lib.ls_head_norm_gate, (
             c_int(DTYPE_CODE[out.dtype]), _ptr(x), c_long(x.stride(0)), c_int(x.shape[0]), c_int(heads), c_int(vdim),
-            _ptr(weight), _ptr(gate), c_long(ldg), c_int(int(gate_act == "sigmoid")), c_float(eps), _ptr(out),
+            _ptr(weight), c_int(each), _ptr(gate), c_long(ldg), c_int(int(gate_act == "sigmoid")), _ptr(denom), c_float(denom_eps),
+            c_float(eps), _ptr(out),
             c_long(out.stride(0)), _stream()))
 
 
@@ -994,7 +1001,7 @@ class Kernels:
     def qkv_post(self, raw: torch.Tensor, n_tokens: int, heads: int, kv_heads: int, dim: int, vdim: int, bias, q_norm,
                  k_norm, eps: float, cos, sin, rot: int, neighbours: bool, max_pos: int, tok_seq, tok_pos, seqs, table,
                  q_out: torch.Tensor, k_pages, v_pages, page_size: int, keys_are_values: bool = False,
-                 key_pad: int | None = None, per_head: bool = False, head_weights: bool = False) -> None:
+                 key_pad: int | None = None, per_head: bool = False, head_weights: bool = False, value_scale: float = 1.0) -> None:
         """Post pass of the fused projection ``raw`` (float32, ``q | k | v | ...``; no ``v`` with
         ``keys_are_values``, where the biased, unnormalised keys are stored as the values): biases, a
         root-mean-square norm over the whole of q and of k with the weights ``q_norm`` / ``k_norm``, rotation of
@@ -1002,7 +1009,8 @@ class Kernels:
         ``q_out``, keys and values to their pages.  ``key_pad``: the size of a head in ``q_out`` and in the key
         pages where it exceeds ``dim`` (zeros beyond ``dim``).  ``per_head``: every head of q and of k is divided
         by its own root mean square over ``dim`` (``eps`` inside the root, no weights) instead; with
-        ``head_weights`` as well, then multiplied by ``q_norm`` / ``k_norm`` of ``dim`` elements, which all heads share."""
+        ``head_weights`` as well, then multiplied by ``q_norm`` / ``k_norm`` of ``dim`` elements, which all heads share.
+        Values are stored times ``value_scale``."""
         _rows_ok(raw, "qkv_post raw"); _rows_ok(q_out, "qkv_post q_out")
         key_pad = dim if key_pad is None else key_pad
         width = heads * dim + kv_heads * dim + (0 if keys_are_values else kv_heads * vdim)
@@ -1038,7 +1046,7 @@ class Kernels:
             c_int(kv_heads), c_int(dim), c_int(key_pad), c_int(vdim), c_int(int(keys_are_values)), c_int(2 if head_weights else int(per_head)), _ptr(bias), _ptr(q_norm), _ptr(k_norm),
             c_float(eps), _ptr(cos), _ptr(sin), c_int(rot), c_int(int(neighbours)), c_int(positions), c_int(max_pos),
             _ptr(tok_seq), _ptr(tok_pos), _ptr(seqs), _ptr(table), c_int(table.shape[1]), _ptr(q_out),
-            c_long(q_out.stride(0)), _ptr(k_pages), _ptr(v_pages), c_int(page_size), _stream()))
+            c_long(q_out.stride(0)), _ptr(k_pages), _ptr(v_pages), c_int(page_size), c_float(value_scale), _stream()))
 
     def sink_attention(self, q: torch.Tensor, heads: int, kv_heads: int, dim: int, vdim: int, k_pages, v_pages,
                        page_size: int, table, seqs, items: torch.Tensor, n_items: int, row_tiles: int, scale: float,
@@ -1128,16 +1136,24 @@ class Kernels:
 
     def experts_route(self, logits: torch.Tensor, bias, top: int, rows_a_tile: int, expert: torch.Tensor,
                       weight: torch.Tensor, order: torch.Tensor, tiles: torch.Tensor, counts: torch.Tensor,
-                      scoring: str = "softmax") -> None:
+                      scoring: str = "softmax", correction=None, groups: tuple[int, int] = (1, 1)) -> None:
         """From router ``logits [T, E]`` (float32) and ``bias [E]``: every token's ``top`` experts (largest logit
         first, the lower index wins a tie) into ``expert [T, top]``, the softmax over the chosen logits into
         ``weight [T, top]``; the pairs ``token * top + choice`` sorted by expert into ``order``, and every
         expert's pairs cut into ``tiles [capacity, 4]`` (expert or -1, first place in ``order``, rows, 0).
-        ``scoring = "sigmoid"``: every chosen expert weighs the sigmoid of its own logit instead (the weights of a token need not add up to one)."""
+        ``scoring = "sigmoid"``: every chosen expert weighs the sigmoid of its own logit instead (the weights of a token need not add up to one).
+        ``scoring = "softmax_all"``: scores are the softmax over all logits; the choice goes by score + ``correction [E]``, within
+        the ``groups[1]`` best of ``groups[0]`` equal runs of neighbouring experts (a run counts by its largest choice
+        score); the weights are the chosen experts' scores divided by their sum."""
         _rows_ok(logits, "experts_route logits")
-        if scoring not in ("softmax", "sigmoid"):
-            raise KernelError(f"experts_route: scoring is softmax or sigmoid, got {scoring!r}")
+        if scoring not in ("softmax", "sigmoid", "softmax_all"):
+            raise KernelError(f"experts_route: scoring is softmax, sigmoid or softmax_all, got {scoring!r}")
         t, e = logits.shape
+        count, keep = groups
+        if scoring == "softmax_all":
+            self._f32_vector(correction, e, "experts_route correction")
+            if not (0 < keep <= count and e % count == 0 and top <= keep * (e // count)):
+                raise KernelError(f"experts_route: {e} experts in {count} groups of which {keep} are kept, {top} a token")
         if not (logits.dtype == torch.float32 and 0 < top <= min(e, self.experts_max_top())):
             raise KernelError(f"experts_route: float32 logits and 1 <= top <= {min(e, self.experts_max_top())}, got {top}")
         if bias is not None:
@@ -1152,13 +1168,13 @@ class Kernels:
         lib = self.experts_lib()
         self._launch(lib, lib.ls_experts_route, (
             _ptr(logits), c_long(logits.stride(0)), _ptr(bias), c_int(t), c_int(e), c_int(top), c_int(rows_a_tile),
-            _ptr(expert), _ptr(weight), _ptr(order), _ptr(tiles), c_int(cap), _ptr(counts), c_int(int(scoring == "sigmoid")),
-            _stream()))
+            _ptr(expert), _ptr(weight), _ptr(order), _ptr(tiles), c_int(cap), _ptr(counts), c_int(("softmax", "sigmoid", "softmax_all").index(scoring)),
+            _ptr(correction), c_int(count), c_int(keep), _stream()))
 
     def experts_apply(self, x: torch.Tensor, w_gate: torch.Tensor, w_up: torch.Tensor, w_down: torch.Tensor, top: int,
                       rows_a_tile: int, order: torch.Tensor, tiles: torch.Tensor, weight: torch.Tensor, limit: float,
                       alpha: float, act: torch.Tensor, partials: torch.Tensor, shift: float = 1.0,
-                      weigh_input: bool = False) -> None:
+                      weigh_input: bool = False, identity: int = 0) -> None:
         """``partials[k][t] = weight[t, k] * down_e(act(gate_e x[t], up_e x[t]))`` for every token's ``k``-th
         expert ``e``, with the clamped gated unit of ``glu_clamped`` as activation (``min(g, limit) sigmoid(alpha
         min(g, limit)) (clamp(u, -limit, limit) + shift)``; an infinite ``limit``, ``alpha`` 1 and ``shift`` 0 are the
@@ -1166,7 +1182,7 @@ class Kernels:
         ``[E, F, K]``, ``w_down [E, N, F]`` in the compute dtype; ``act``: scratch ``[T * top, F]`` of the
         compute dtype; ``partials [top, T, N]`` float32; the routing as ``experts_route`` left it.
         ``weigh_input``: the weight multiplies the expert's input instead, ``partials[k][t] = down_e(act(w gate_e
-        x[t], w up_e x[t]))``."""
+        x[t], w up_e x[t]))``.  ``identity``: that many experts behind those with weights return their input."""
         _rows_ok(x, "experts_apply x"); _rows_ok(act, "experts_apply act")
         t, k = x.shape
         if not (w_gate.dim() == 3 and w_gate.shape == w_up.shape and w_gate.shape[2] == k and w_down.dim() == 3
@@ -1174,7 +1190,10 @@ class Kernels:
                 and w_gate.is_contiguous() and w_up.is_contiguous() and w_down.is_contiguous()
                 and w_gate.dtype == x.dtype == w_up.dtype == w_down.dtype == act.dtype and x.dtype in DTYPE_CODE):
             raise KernelError("experts_apply weights must be [E, F, K], [E, F, K], [E, N, F] of the compute dtype")
-        e, f, n = w_gate.shape[0], w_gate.shape[1], w_down.shape[1]
+        real, f, n = w_gate.shape[0], w_gate.shape[1], w_down.shape[1]
+        e = real + identity
+        if not (identity >= 0 and (identity == 0 or n == k)):
+            raise KernelError(f"experts_apply: an expert that returns its input of {k} elements cannot stand beside outputs of {n}")
         cap = self.experts_tile_capacity(t, e, top, rows_a_tile)
         if not (act.shape[0] >= t * top and act.shape[1] == f):
             raise KernelError(f"experts_apply act must be [>= {t * top}, {f}]")
@@ -1191,7 +1210,7 @@ class Kernels:
             c_int(DTYPE_CODE[x.dtype]), _ptr(x), c_long(x.stride(0)), _ptr(w_gate), _ptr(w_up), _ptr(w_down), c_int(t),
             c_int(e), c_int(top), c_int(k), c_int(f), c_int(n), c_int(rows_a_tile), _ptr(order), _ptr(tiles), c_int(cap),
             _ptr(weight), c_float(limit), c_float(alpha), c_float(shift), _ptr(act), c_long(act.stride(0)), _ptr(partials),
-            c_int(int(bool(weigh_input))), _stream()))
+            c_int(int(bool(weigh_input))), c_int(real), _stream()))
 
     def experts_route_table(self, token_ids: torch.Tensor, table: torch.Tensor, experts: int, rows_a_tile: int,
                             expert: torch.Tensor, weight: torch.Tensor, order: torch.Tensor, tiles: torch.Tensor,
@@ -1224,12 +1243,12 @@ class Kernels:
                                                      int(self.mixers_lib().ls_streams_max_width())))
 
     def streams_step(self, x: torch.Tensor, copies: int, partials, mix, gain, take, weight, eps: float, out,
-                     rows: torch.Tensor | None = None) -> None:
+                     rows: torch.Tensor | None = None, bias=None, centred: bool = False) -> None:
         """One step of a residual stream of ``copies`` copies, ``x`` float32 ``[T, copies * width]``.  With
         ``partials [slices, T, width]`` (a sublayer's output as slice sums) the copies are rewritten:
         ``x'_t = sum_s mix[s, t] x_s + gain[t] y``, ``y`` the sum of the slices in ascending order.  With ``out
         [rows, width]`` the copies are then read: ``u = sum_t take[t] x'_t`` (``take`` None: their plain sum) and
-        ``out = u / sqrt(mean(u^2) + eps) * weight``.  ``rows`` selects rows of ``x`` (all without it)."""
+        ``out = (u - m) / sqrt(mean((u - m)^2) + eps) * weight (+ bias)`` with ``m`` the row's mean if ``centred``, else 0.  ``rows`` selects rows of ``x`` (all without it)."""
         _rows_ok(x, "streams_step x")
         if not (x.dtype == torch.float32 and copies > 0 and x.shape[1] % copies == 0):
             raise KernelError("streams_step works on float32 rows of whole copies")
@@ -1255,6 +1274,8 @@ class Kernels:
             if not (out.dtype in DTYPE_CODE and tuple(out.shape) == (n_rows, width) and eps > 0):
                 raise KernelError(f"streams_step out must be [{n_rows},{width}], eps positive")
             self._f32_vector(weight, width, "streams_step weight")
+            if bias is not None:
+                self._f32_vector(bias, width, "streams_step bias")
             dtype, ld_out = out.dtype, out.stride(0)
         elif partials is None:
             return
@@ -1263,7 +1284,8 @@ class Kernels:
         lib = self.mixers_lib()
         self._launch(lib, lib.ls_streams_step, (
             c_int(DTYPE_CODE[dtype]), _ptr(x), c_long(x.stride(0)), c_int(copies), c_int(width), _ptr(partials),
-            c_int(slices), c_int(p_rows), _ptr(mix), _ptr(gain), _ptr(take), _ptr(weight), c_float(eps), _ptr(out),
+            c_int(slices), c_int(p_rows), _ptr(mix), _ptr(gain), _ptr(take), _ptr(weight), _ptr(bias), c_int(int(centred)),
+            c_float(eps), _ptr(out),
             c_long(ld_out), _ptr(rows), c_int(n_rows), _stream()))
 
     # -- attention over a cached latent: the passes around it ----------------------------------------
@@ -1502,7 +1524,7 @@ class Kernels:
         width]`` (a sublayer's output as slice sums, added in ascending order to ``y``): ``x += y``, or, with ``post``,
         ``x += norm(y)``.  With ``results [layers + 1, T, width]``: ``results[keep] = x``; with ``shares [keep + 1]`` then
         ``x = sum_j shares[j] results[j]``.  With ``out [rows, width]``: ``out = norm(x)``.  ``post`` and ``norm`` are
-        ``(weight, eps, centred)``; a norm is ``(v - m) / sqrt(mean((v - m)^2) + eps) * weight`` with ``m`` the row's mean
+        ``(weight, eps, centred)``, ``norm`` with an optional fourth entry, a bias (or None) that is added behind it; a norm is ``(v - m) / sqrt(mean((v - m)^2) + eps) * weight`` with ``m`` the row's mean
         if ``centred``, else 0.  ``rows`` selects rows of ``x``; then nothing but ``out`` is written."""
         _rows_ok(x, "residual_step x")
         t, width = x.shape
@@ -1519,7 +1541,9 @@ class Kernels:
                     and partials.shape[2] == width and partials.shape[1] >= t):
                 raise KernelError(f"residual_step partials must be float32 [slices, >= {t}, {width}]")
             slices, p_rows = partials.shape[0], partials.shape[1]
-        post_weight, post_eps, post_centred = post if post is not None else (None, 0.0, False)
+        post_weight, post_eps, post_centred = tuple(post)[:3] if post is not None else (None, 0.0, False)
+        if post is not None and len(post) > 3 and post[3] is not None:
+            raise KernelError("residual_step: a norm of the sublayer's output has no bias")
         if post is not None:
             if partials is None:
                 raise KernelError("residual_step: a norm of the sublayer's output needs its slices")
@@ -1533,9 +1557,11 @@ class Kernels:
             if results is None:
                 raise KernelError("residual_step: shares need results")
             self._f32_vector(shares, keep + 1, "residual_step shares")
-        weight, eps, centred, dtype, ld_out = None, 0.0, False, torch.float32, 0
+        weight, eps, centred, bias, dtype, ld_out = None, 0.0, False, None, torch.float32, 0
         if out is not None:
-            weight, eps, centred = norm
+            weight, eps, centred, bias = (tuple(norm) + (None,))[:4]
+            if bias is not None:
+                self._f32_vector(bias, width, "residual_step bias")
             _rows_ok(out, "residual_step out")
             if not (out.dtype in DTYPE_CODE and tuple(out.shape) == (n_rows, width) and eps > 0):
                 raise KernelError(f"residual_step out must be [{n_rows},{width}], eps positive")
@@ -1548,7 +1574,7 @@ class Kernels:
         self._launch(lib, lib.ls_residual_step, (
             c_int(DTYPE_CODE[dtype]), _ptr(x), c_long(x.stride(0)), c_int(width), _ptr(partials), c_int(slices), c_int(p_rows),
             _ptr(post_weight), c_float(post_eps), c_int(int(post_centred)), _ptr(results), c_int(r_rows), c_int(keep),
-            _ptr(shares), _ptr(weight), c_float(eps), c_int(int(centred)), _ptr(out), c_long(ld_out), _ptr(rows), c_int(n_rows),
+            _ptr(shares), _ptr(weight), _ptr(bias), c_float(eps), c_int(int(centred)), _ptr(out), c_long(ld_out), _ptr(rows), c_int(n_rows),
             _stream()))
 
     def channel_recurrence(self, raw: torch.Tensor, a_at: int, u_at: int, g_at: int, a_bias, u_bias, seqs, n_seqs: int,
@@ -1594,6 +1620,199 @@ class Kernels:
         self._launch(lib, lib.ls_embed_positions, (
             c_int(DTYPE_CODE[table.dtype]), _ptr(tokens), _ptr(tok_pos), _ptr(table), c_int(table.shape[0]), _ptr(freq),
             _ptr(out), c_int(t), c_int(width), c_long(out.stride(0)), c_float(scale), _stream()))
+
+    # -- matrix memories with one gate a head and token ------------------------------------------------
+    #: floats of a head's gates of a token (log a, b, floor, n . q)
+    GATE_FLOATS = 4
+
+    def memory_max_rows(self) -> int:
+        return self._memo(("memory_max_rows",), lambda: int(self.mixers_lib().ls_memory_max_rows()))
+
+    def memory_chunk(self) -> int:
+        """Tokens of a chunk of ``memory_chunks``."""
+        return self._memo(("memory_chunk",), lambda: int(self.mixers_lib().ls_memory_chunk()))
+
+    def _memory_state(self, state, floats: int, what: str) -> None:
+        if not (state.is_cuda and state.dtype == torch.float32 and state.dim() == 2 and state.stride(1) == 1 and state.shape[1] >= floats):
+            raise KernelError(f"{what} state must be float32 [slots, >= {floats}]")
+
+    def _gates_ok(self, gates, n_tokens: int, heads: int, what: str) -> None:
+        if not (gates.is_cuda and gates.dtype == torch.float32 and gates.is_contiguous()
+                and gates.numel() >= n_tokens * heads * self.GATE_FLOATS):
+            raise KernelError(f"{what} gates: float32, four a token and head")
+
+    def _tokens_ok(self, n_tokens: int, tok_seq, tok_pos, what: str) -> None:
+        for name, v in (("tok_seq", tok_seq), ("tok_pos", tok_pos)):
+            if not (v.is_cuda and v.dtype == torch.int32 and v.is_contiguous() and v.numel() >= n_tokens):
+                raise KernelError(f"{what} {name}: int32, one entry a token")
+
+    def _seqs_ok(self, seqs, n_seqs: int, what: str) -> None:
+        self._i32(seqs, 8 * n_seqs, f"{what} seqs")
+
+    def _space_ok(self, raw, x_at, dt_at, channels, heads, taps, conv_bias, a_log, dt_bias, what: str) -> int:
+        _rows_ok(raw, f"{what} raw")
+        if not (raw.dtype == torch.float32 and min(x_at, dt_at) >= 0 and raw.shape[1] >= max(x_at + channels, dt_at + heads)):
+            raise KernelError(f"{what}: the projections do not fit the float32 rows")
+        if not (taps.is_cuda and taps.dtype == torch.float32 and taps.is_contiguous() and taps.dim() == 2
+                and taps.shape[1] == channels and taps.shape[0] >= 1):
+            raise KernelError(f"{what} taps must be float32 [M, {channels}]")
+        self._f32_vector(conv_bias, channels, f"{what} conv bias")
+        self._f32_vector(a_log, heads, f"{what} a_log")
+        self._f32_vector(dt_bias, heads, f"{what} dt_bias")
+        return taps.shape[0]
+
+    def conv_gates(self, raw: torch.Tensor, x_at: int, dt_at: int, channels: int, heads: int, taps: torch.Tensor, conv_bias, a_log,
+                   dt_bias, tok_seq, tok_pos, seqs, n_seqs: int, state: torch.Tensor, ring_at: int, conv: torch.Tensor,
+                   gates: torch.Tensor) -> None:
+        """What a state-space mixer computes of a step's tokens before its memory.  Every one of the ``channels`` columns of
+        the float32 rows ``raw`` from ``x_at`` on passes ``silu(bias + sum_m taps[m] in(p - M + 1 + m))`` into ``conv [T,
+        channels]``; ``dt = softplus(raw[dt_at ..] + dt_bias)`` gives the gates ``log a = -exp(a_log) dt``, ``b = dt``.  ``taps [M,
+        channels]``.  ``state``: at ``ring_at`` the ring ``[M, channels]`` of the request's last inputs, which this call moves on."""
+        m = self._space_ok(raw, x_at, dt_at, channels, heads, taps, conv_bias, a_log, dt_bias, "conv_gates")
+        t = raw.shape[0]
+        self._memory_state(state, ring_at + m * channels, "conv_gates")
+        self._gates_ok(gates, t, heads, "conv_gates")
+        self._tokens_ok(t, tok_seq, tok_pos, "conv_gates")
+        self._seqs_ok(seqs, n_seqs, "conv_gates")
+        if not (conv.is_cuda and conv.dtype == torch.float32 and conv.is_contiguous() and tuple(conv.shape) == (t, channels)):
+            raise KernelError(f"conv_gates conv must be float32 [{t}, {channels}]")
+        if t == 0:
+            return
+        lib = self.mixers_lib()
+        self._launch(lib, lib.ls_conv_gates, (
+            _ptr(raw), c_long(raw.stride(0)), c_int(x_at), c_int(dt_at), c_int(t), c_int(channels), c_int(heads), c_int(m), _ptr(taps),
+            _ptr(conv_bias), _ptr(a_log), _ptr(dt_bias), _ptr(tok_seq), _ptr(tok_pos), _ptr(seqs), c_int(n_seqs), _ptr(state),
+            c_long(state.stride(0)), c_long(ring_at), _ptr(conv), _ptr(gates), _stream()))
+
+    def exp_gates(self, raw: torch.Tensor, i_at: int, f_at: int, heads: int, i_bias, f_bias, cap: float, seqs, n_seqs: int,
+                  state: torch.Tensor, max_at: int, gates: torch.Tensor) -> None:
+        """Exponential gates: ``i = cap tanh((raw[i_at ..] + i_bias) / cap)``, ``f = logsigmoid(cap tanh((raw[f_at ..] + f_bias) /
+        cap))``, a running maximum ``m = max(f + m, i)`` from zero; ``log a = f + m_before - m``, ``b = exp(i - m)``, floor
+        ``exp(-m)``.  ``state``: at ``max_at`` two numbers a head, of which the one of the length's parity is the maximum."""
+        _rows_ok(raw, "exp_gates raw")
+        if not (raw.dtype == torch.float32 and cap > 0 and min(i_at, f_at) >= 0 and raw.shape[1] >= max(i_at, f_at) + heads):
+            raise KernelError("exp_gates: the projections do not fit the float32 rows, or the cap is not positive")
+        self._f32_vector(i_bias, heads, "exp_gates i_bias"); self._f32_vector(f_bias, heads, "exp_gates f_bias")
+        self._memory_state(state, max_at + 2 * heads, "exp_gates")
+        self._gates_ok(gates, raw.shape[0], heads, "exp_gates")
+        self._seqs_ok(seqs, n_seqs, "exp_gates")
+        if raw.shape[0] == 0:
+            return
+        lib = self.mixers_lib()
+        self._launch(lib, lib.ls_exp_gates, (
+            _ptr(raw), c_long(raw.stride(0)), c_int(i_at), c_int(f_at), c_int(heads), _ptr(i_bias), _ptr(f_bias), c_float(cap),
+            _ptr(seqs), c_int(n_seqs), _ptr(state), c_long(state.stride(0)), c_long(max_at), _ptr(gates), _stream()))
+
+    def _memory_rows(self, rows, heads: int, size: int, n_tokens: int, what: str):
+        """``rows``: (float32 rows, column of head 0, heads that share one) of q, k or v; their pointer, strides and share."""
+        t, at, share = rows
+        _rows_ok(t, what)
+        if not (t.dtype == torch.float32 and share > 0 and heads % share == 0 and at >= 0 and t.shape[0] >= n_tokens
+                and t.shape[1] >= at + (heads // share) * size):
+            raise KernelError(f"{what}: {heads // max(share, 1)} heads of {size} do not fit the float32 rows")
+        return c_void_p(t.data_ptr() + 4 * at), c_long(t.stride(0)), c_int(size), c_int(share)
+
+    def memory(self, q, k, v, gates: torch.Tensor, heads: int, rows: int, vdim: int, q_scale: float, skip, norm: bool, seqs,
+               n_seqs: int, longest: int, walks: bool, items, n_items: int, runs, n_runs: int, states, decays, state: torch.Tensor,
+               out: torch.Tensor) -> None:
+        """A matrix memory over the tokens of every request of the step: per head ``S <- a S + b k v^T`` (``rows x vdim``),
+        ``out = S^T q * q_scale + skip v``; with ``norm`` also ``n <- a n + b k`` and ``n . q`` into the gates' last place.  ``q``,
+        ``k``, ``v``: (float32 rows ``[T, .]``, first column, heads that share one); ``gates`` as ``conv_gates`` or ``exp_gates``
+        left them.  Requests of at most ``longest`` tokens walk token by token (``walks``: there are some); the others go
+        by chunks of ``memory_chunk()`` tokens: ``items`` (request of the step, chunk) and ``runs`` (request, first item,
+        items, 0) name them, ``states [n_items, floats]`` and ``decays [n_items, heads]`` are scratch.  ``state [slots, .]``: ``S``,
+        then ``n``."""
+        t = out.shape[0]
+        floats = heads * rows * vdim + (heads * rows if norm else 0)
+        if not (0 < rows <= self.memory_max_rows()):
+            raise KernelError(f"memory: states of at most {self.memory_max_rows()} rows a head, got {rows}")
+        _rows_ok(out, "memory out")
+        if not (out.dtype == torch.float32 and out.shape[1] == heads * vdim):
+            raise KernelError(f"memory out must be float32 [T, {heads * vdim}]")
+        self._memory_state(state, floats, "memory")
+        self._gates_ok(gates, t, heads, "memory")
+        self._seqs_ok(seqs, n_seqs, "memory")
+        if skip is not None:
+            self._f32_vector(skip, heads, "memory skip")
+        if v[2] != 1:
+            raise KernelError("memory: every head has values of its own")
+        qa = self._memory_rows(q, heads, rows, t, "memory q")
+        ka = self._memory_rows(k, heads, rows, t, "memory k")
+        va = self._memory_rows(v, heads, vdim, t, "memory v")[:3]
+        if n_items:
+            self._i32(items, 2 * n_items, "memory items"); self._i32(runs, 4 * n_runs, "memory runs")
+            for name, s, n in (("states", states, n_items * floats), ("decays", decays, n_items * heads)):
+                if not (s is not None and s.is_cuda and s.dtype == torch.float32 and s.is_contiguous() and s.numel() >= n):
+                    raise KernelError(f"memory {name}: float32 scratch of {n} elements")
+        if t == 0:
+            return
+        lib = self.mixers_lib()
+        head = (*qa, *ka, *va, _ptr(gates), c_int(heads), c_int(rows), c_int(vdim), c_float(q_scale), _ptr(skip), c_int(int(norm)),
+                _ptr(seqs))
+        tail = (_ptr(state), c_long(state.stride(0)), _ptr(out), c_long(out.stride(0)), _stream())
+        if walks:
+            self._launch(lib, lib.ls_memory_walk, (*head, c_int(n_seqs), c_int(longest), *tail))
+        if n_items:
+            self._launch(lib, lib.ls_memory_chunks, (*head, _ptr(items), c_int(n_items), _ptr(runs), c_int(n_runs), _ptr(states),
+                                                     c_long(floats), _ptr(decays), *tail))
+
+    def space_token(self, raw: torch.Tensor, x_at: int, dt_at: int, groups: int, taps: torch.Tensor, conv_bias, a_log, dt_bias, skip,
+                    heads: int, rows: int, vdim: int, seqs, n_seqs: int, state: torch.Tensor, ring_at: int, out: torch.Tensor) -> None:
+        """A step of single tokens of a state-space mixer in one launch: what ``conv_gates`` and ``memory`` do (channels ``x``
+        (heads x vdim) ``| B | C`` (groups x rows each) from ``x_at`` on)."""
+        channels = heads * vdim + 2 * groups * rows
+        m = self._space_ok(raw, x_at, dt_at, channels, heads, taps, conv_bias, a_log, dt_bias, "space_token")
+        self._f32_vector(skip, heads, "space_token skip")
+        self._memory_state(state, ring_at + m * channels, "space_token")
+        self._seqs_ok(seqs, n_seqs, "space_token")
+        _rows_ok(out, "space_token out")
+        if not (out.dtype == torch.float32 and tuple(out.shape) == (n_seqs, heads * vdim) and raw.shape[0] >= n_seqs and heads % groups == 0):
+            raise KernelError(f"space_token out must be float32 [{n_seqs}, {heads * vdim}], heads a multiple of the groups")
+        if n_seqs == 0:
+            return
+        lib = self.mixers_lib()
+        self._launch(lib, lib.ls_space_token, (
+            _ptr(raw), c_long(raw.stride(0)), c_int(x_at), c_int(dt_at), c_int(channels), c_int(groups), c_int(m), c_long(ring_at),
+            _ptr(taps), _ptr(conv_bias), _ptr(a_log), _ptr(dt_bias), _ptr(skip), c_int(heads), c_int(rows), c_int(vdim), _ptr(seqs),
+            c_int(n_seqs), _ptr(state), c_long(state.stride(0)), _ptr(out), c_long(out.stride(0)), _stream()))
+
+    def exp_token(self, raw: torch.Tensor, q_at: int, k_at: int, v_at: int, i_at: int, f_at: int, i_bias, f_bias, cap: float,
+                  q_scale: float, heads: int, rows: int, vdim: int, seqs, n_seqs: int, state: torch.Tensor, max_at: int,
+                  gates: torch.Tensor, out: torch.Tensor) -> None:
+        """A step of single tokens of a memory with exponential gates in one launch: what ``exp_gates`` and ``memory`` do."""
+        _rows_ok(raw, "exp_token raw"); _rows_ok(out, "exp_token out")
+        if not (raw.dtype == torch.float32 and cap > 0 and min(q_at, k_at, v_at, i_at, f_at) >= 0 and raw.shape[0] >= n_seqs
+                and raw.shape[1] >= max(max(q_at, k_at) + heads * rows, v_at + heads * vdim, max(i_at, f_at) + heads)):
+            raise KernelError("exp_token: the projections do not fit the float32 rows, or the cap is not positive")
+        self._f32_vector(i_bias, heads, "exp_token i_bias"); self._f32_vector(f_bias, heads, "exp_token f_bias")
+        self._memory_state(state, max_at + 2 * heads, "exp_token")
+        self._gates_ok(gates, n_seqs, heads, "exp_token")
+        self._seqs_ok(seqs, n_seqs, "exp_token")
+        if not (out.dtype == torch.float32 and tuple(out.shape) == (n_seqs, heads * vdim)):
+            raise KernelError(f"exp_token out must be float32 [{n_seqs}, {heads * vdim}]")
+        if n_seqs == 0:
+            return
+        lib = self.mixers_lib()
+        self._launch(lib, lib.ls_exp_token, (
+            _ptr(raw), c_long(raw.stride(0)), c_int(q_at), c_int(k_at), c_int(v_at), c_int(i_at), c_int(f_at), c_long(max_at),
+            _ptr(i_bias), _ptr(f_bias), c_float(cap), c_float(q_scale), c_int(heads), c_int(rows), c_int(vdim), _ptr(seqs),
+            c_int(n_seqs), _ptr(state), c_long(state.stride(0)), _ptr(gates), _ptr(out), c_long(out.stride(0)), _stream()))
+
+    def gated_parts_norm(self, y: torch.Tensor, z: torch.Tensor, parts: int, weight, eps: float, out: torch.Tensor) -> None:
+        """``y * silu(z)``, divided by its root mean square in each of ``parts`` equal runs of a row (``eps`` inside the
+        root), times ``weight``; ``y`` and ``z`` float32 rows."""
+        _rows_ok(y, "gated_parts_norm y"); _rows_ok(z, "gated_parts_norm z"); _rows_ok(out, "gated_parts_norm out")
+        t, inner = out.shape
+        if not (y.dtype == torch.float32 and z.dtype == torch.float32 and tuple(y.shape) == (t, inner) and tuple(z.shape) == (t, inner)
+                and out.dtype in DTYPE_CODE and parts > 0 and inner % parts == 0 and eps > 0):
+            raise KernelError(f"gated_parts_norm: float32 rows of {inner} elements in {parts} equal parts, eps positive")
+        self._f32_vector(weight, inner, "gated_parts_norm weight")
+        if t == 0:
+            return
+        lib = self.mixers_lib()
+        self._launch(lib, lib.ls_gated_parts_norm, (
+            c_int(DTYPE_CODE[out.dtype]), _ptr(y), c_long(y.stride(0)), _ptr(z), c_long(z.stride(0)), c_int(t), c_int(inner),
+            c_int(parts), _ptr(weight), c_float(eps), _ptr(out), c_long(out.stride(0)), _stream()))
 
 
 ATTENTION_ITEM_INTS = 32

@@ -170,6 +170,10 @@ class Mixer(Part):
         """``PagedKVSpec``, ``StateSpec`` or ``None``."""
         return None
 
+    def further_specs(self) -> tuple:
+        """What a mixer keeps beside ``cache_spec()``: a spec for every unit of its schedule entries' ``further``."""
+        return ()
+
     def prepare(self, ctx) -> None:
         """Declare per-step needs (work lists) before the step's metadata is uploaded."""
 
@@ -185,6 +189,40 @@ class Mixer(Part):
 
     def forward(self, ctx, run, x, out, accumulate: bool) -> None:
         raise NotImplementedError
+
+
+class ProjectedMixer(Mixer):
+    """A mixer of the form ``out (+)= W_out mix(W_in x)``: one product of the tokens' rows, stored in float32, then ``mix``
+    (attention, a recurrence, ...), whose rows in the compute dtype are the operand of the output product.  A part
+    that runs several such mixers on the same input forms both products for all of them at once
+    (``side_by_side``); so what belongs to the products is kept apart from the rest.  The parameter ``out_scale``
+    (default 1) multiplies what ``mix`` leaves."""
+
+    #: columns of what ``mix`` leaves
+    out_width = 0
+
+    def in_matrices(self, weights) -> list:
+        """The tensors whose rows, one below the other, are ``W_in``."""
+        raise NotImplementedError
+
+    def out_matrix(self, weights):
+        raise NotImplementedError
+
+    def load_own(self, weights, rt) -> None:
+        """Everything but the two products' matrices."""
+
+    def mix(self, ctx, run, raw, out) -> None:
+        """From the float32 rows ``raw`` of the input product to the rows ``out [T, out_width]`` of the compute dtype."""
+        raise NotImplementedError
+
+
+def stack_rows(tensors):
+    """One matrix of the tensors' rows (in float32 if their dtypes differ)."""
+    import torch
+
+    if len({t.dtype for t in tensors}) > 1:
+        tensors = [t.to(torch.float32) for t in tensors]
+    return torch.cat(tensors, dim=0)
 
 
 class FeedForward(Part):

@@ -2,6 +2,8 @@
 
 from __future__ import annotations
 
+import torch
+
 from .base import Arrangement, PendingAdd, StateSpec, WeightSpec, build_part, register_part, takes
 
 
@@ -198,7 +200,10 @@ class HyperConnections(Arrangement):
     Parameters: ``copies``; ``mixer_prefix``, ``feed_forward_prefix``, ``mixer_norm_name``,
     ``feed_forward_norm_name`` as for ``prenorm_residual``; ``mixer_streams_prefix``,
     ``feed_forward_streams_prefix``: below them the tensors ``in [n]`` (take), ``out [n]`` (gain) and
-    ``mix [n, n]``.  The norms must be ``rmsnorm`` parts (their weight and eps are applied by the read)."""
+    ``mix [n, n]``.  The norms must be ``rmsnorm`` or ``layernorm`` parts (the read applies them).
+
+    ``residual_mult`` (default 1): what a sublayer returns is written times this number.  ``learned`` (default True):
+    False for a layer without such tensors, over one copy: ``x' = x + residual_mult y``."""
 
     graph_safe = True
 
@@ -209,6 +214,10 @@ class HyperConnections(Arrangement):
         self.copies = int(p["copies"])
         if self.copies < 1:
             raise ValueError(f"a residual stream of {self.copies} copies")
+        self.mult = 1.0 if p.get("residual_mult") is None else float(p["residual_mult"])
+        self.learned = p.get("learned", True) is not False
+        if not self.learned and self.copies != 1:
+            raise ValueError(f"a residual stream of {self.copies} copies needs the tensors that mix them")
         self.mixer_norm = build_part(layer_spec.part("mixer_norm"), self.join(base, p["mixer_norm_name"]))
         self._mixer = build_part(layer_spec.part("mixer"), self.join(base, p["mixer_prefix"]))
         self.feed_forward = self.feed_forward_norm = None
@@ -217,8 +226,8 @@ class HyperConnections(Arrangement):
                                                 self.join(base, p["feed_forward_norm_name"]))
             self.feed_forward = build_part(layer_spec.part("feed_forward"), self.join(base, p["feed_forward_prefix"]))
         for norm in (self.mixer_norm, self.feed_forward_norm):
-            if norm is not None and getattr(norm, "kind", "") != "rmsnorm":
-                raise ValueError("the sublayers of a stream of several copies are normalised by rmsnorm parts")
+            if norm is not None and getattr(norm, "kind", "") not in ("rmsnorm", "layernorm"):
+                raise ValueError("the sublayers of a stream of several copies are normalised by rmsnorm or layernorm parts")
         self._defer_mixer = takes(self._mixer.forward, "defer")
         self._defer_ff = self.feed_forward is not None and takes(self.feed_forward.forward, "defer")
         self.streams = {}        # sublayer -> (take, gain, mix) on the device
@@ -238,17 +247,21 @@ class HyperConnections(Arrangement):
         p = layer_spec.arrangement.params
         base, n = layer_spec.prefix, int(p["copies"])
         out = []
+        learned = p.get("learned", True) is not False
         wired = [(layer_spec.part("mixer_norm"), p["mixer_norm_name"]), (layer_spec.part("mixer"), p["mixer_prefix"])]
-        out += cls._stream_specs(cls.join(base, p["mixer_streams_prefix"]), n)
+        if learned:
+            out += cls._stream_specs(cls.join(base, p["mixer_streams_prefix"]), n)
         if layer_spec.has("feed_forward"):
             wired += [(layer_spec.part("feed_forward_norm"), p["feed_forward_norm_name"]),
                       (layer_spec.part("feed_forward"), p["feed_forward_prefix"])]
-            out += cls._stream_specs(cls.join(base, p["feed_forward_streams_prefix"]), n)
+            if learned:
+                out += cls._stream_specs(cls.join(base, p["feed_forward_streams_prefix"]), n)
         else:
             # what the checkpoint may hold for a second half that never runs is accepted, never used
             if layer_spec.has("feed_forward_norm"):
                 wired.append((layer_spec.part("feed_forward_norm"), p["feed_forward_norm_name"]))
-            out += cls._stream_specs(cls.join(base, p["feed_forward_streams_prefix"]), n, optional=True)
+            if learned:
+                out += cls._stream_specs(cls.join(base, p["feed_forward_streams_prefix"]), n, optional=True)
         for spec, name in wired:
             out += part_class(spec.kind).weight_specs(spec, cls.join(base, name))
         return out
@@ -269,12 +282,19 @@ class HyperConnections(Arrangement):
         most, widest = rt.kernels.streams_max()
         if self.copies > most:
             raise ValueError(f"a residual stream of {self.copies} copies; the kernel takes up to {most}")
-        names = [("mixer", p["mixer_streams_prefix"])]
-        if self.feed_forward is not None:
-            names.append(("feed_forward", p["feed_forward_streams_prefix"]))
-        for sublayer, name in names:
-            full = self.join(self.layer_spec.prefix, name)
-            self.streams[sublayer] = tuple(rt.vector(weights.get(f"{full}.{t}").reshape(-1)) for t in ("in", "out", "mix"))
+        for sublayer in ("mixer",) + (("feed_forward",) if self.feed_forward is not None else ()):
+            if self.learned:
+                full = self.join(self.layer_spec.prefix, p[f"{sublayer}_streams_prefix"])
+                take, gain, mix = (rt.vector(weights.get(f"{full}.{t}").reshape(-1)) for t in ("in", "out", "mix"))
+            else:
+                take, gain, mix = (torch.ones(1, dtype=torch.float32, device=rt.device) for _ in range(3))
+            self.streams[sublayer] = (take, gain * self.mult if self.mult != 1.0 else gain, mix)
+
+    def _read(self, k, h, pending, take, norm, x) -> None:
+        """The pending write into the copies, then ``x = norm(sum_s take[s] x_s)``, in one launch."""
+        weight, eps, centred, bias = (tuple(norm.step_norm()) + (None,))[:4]
+        partials, mix, gain = (None, None, None) if pending is None else (pending.partials, pending.mix, pending.gain)
+        k.streams_step(h, self.copies, partials, mix, gain, take, weight, eps, x, bias=bias, centred=centred)
 
     def forward(self, ctx, run, h, pending=None):
         """``pending``: the write the previous layer left (a ``PendingWrite``).  Returns this layer's last one."""
@@ -287,8 +307,7 @@ class HyperConnections(Arrangement):
             pending = None
         take, gain, mix = self.streams["mixer"]
         x = ctx.buf("block.normed", (ctx.n_tokens, width), rt.dtype)
-        k.streams_step(h, n, None if pending is None else pending.partials, None if pending is None else pending.mix,
-                       None if pending is None else pending.gain, take, self.mixer_norm.weight, self.mixer_norm.eps, x)
+        self._read(k, h, pending, take, self.mixer_norm, x)
         if self._defer_mixer:
             call = lambda y, acc, defer: self._mixer.forward(ctx, run, x, y, accumulate=acc, defer=defer)  # noqa: E731
         else:
@@ -298,8 +317,7 @@ class HyperConnections(Arrangement):
             return left
         take, gain, mix = self.streams["feed_forward"]
         x = ctx.buf("block.normed", (ctx.n_tokens, width), rt.dtype)
-        k.streams_step(h, n, left.partials, left.mix, left.gain, take, self.feed_forward_norm.weight,
-                       self.feed_forward_norm.eps, x)
+        self._read(k, h, left, take, self.feed_forward_norm, x)
         if self._defer_ff:
             call = lambda y, acc, defer: self.feed_forward.forward(ctx, x, y, accumulate=acc, defer=defer)  # noqa: E731
         else:

@@ -10,6 +10,13 @@ With ``score = "sigmoid"`` a chosen expert weighs ``sigmoid(z)`` of its own logi
 (the experts with the largest scores are those with the largest logits).  With ``weigh = "input"`` a weight
 multiplies what its expert reads and not what it returns: ``out[t] = sum_k expert_chosen(t)[k](w[t, k] x[t])``.
 
+With ``score = "softmax_all"`` the scores ``s[t]`` are the softmax over all logits.  The choice goes by ``s + correction`` (a
+learned vector), and only the experts of the best ``groups.keep`` of ``groups.count`` equal runs of neighbours can be chosen (a run
+counts by its largest choice score); the weights are the chosen experts' ``s``, without the correction, divided by their sum.
+
+``identity`` further experts behind those with weights return their input: the router has outputs for them, they count in
+softmax, groups and choice, and they have no tensors.
+
 With ``router = "table"`` there is no router: row ``token id`` of an integer table ``[vocab, top]`` names
 the token's experts (the entries of a row differ) and each weighs ``1 / top``.
 
@@ -43,7 +50,8 @@ class RoutedExperts(FeedForward):
     ``limit`` None: the plain gated unit with SiLU.  ``router`` ``"table"`` (default ``"linear"``): the
     tensor ``table`` ``[vocab_size, top]`` (int) instead of the router's, with the parameter ``vocab_size``.
     ``score`` (``"softmax"`` over the chosen logits, the default, or ``"sigmoid"`` of each), ``weigh`` (``"output"``,
-    the default, or ``"input"``), ``router_bias`` (default True; False: there is no tensor ``router.b``)."""
+    the default, or ``"input"``), ``router_bias`` (default True; False: there is no tensor ``router.b``).  ``score`` ``"softmax_all"`` (with the tensor
+    ``correction [E + identity]``) and ``groups`` (None or ``{"count", "keep"}``) as above; ``identity`` (default 0)."""
 
     graph_safe = True
 
@@ -62,15 +70,24 @@ class RoutedExperts(FeedForward):
             raise ValueError(f"router {p['router']!r} is not one of linear, table")
         self.score, self.weigh = p.get("score") or "softmax", p.get("weigh") or "output"
         self.router_bias = p.get("router_bias", True) is not False
-        if self.score not in ("softmax", "sigmoid") or self.weigh not in ("output", "input"):
-            raise ValueError(f"score {self.score!r} is not softmax or sigmoid, or weigh {self.weigh!r} not output or input")
-        if self.tabled and self.score != "softmax":
-            raise ValueError("experts that a table names have no scores")
-        if not 0 < self.top <= self.experts:
-            raise ValueError(f"a token cannot use {self.top} of {self.experts} experts")
+        if self.score not in ("softmax", "sigmoid", "softmax_all") or self.weigh not in ("output", "input"):
+            raise ValueError(f"score {self.score!r} is not softmax, sigmoid or softmax_all, or weigh {self.weigh!r} not output or input")
+        self.identity = int(p.get("identity") or 0)
+        groups = p.get("groups") or {"count": 1, "keep": 1}
+        self.groups = int(groups["count"]), int(groups["keep"])
+        if self.tabled and (self.score != "softmax" or self.identity):
+            raise ValueError("experts that a table names have no scores, and all of them have weights")
+        self.routed = self.experts + self.identity          # the router's outputs
+        if not 0 < self.top <= self.routed or self.identity < 0:
+            raise ValueError(f"a token cannot use {self.top} of {self.routed} experts")
+        if self.score != "softmax_all" and self.groups != (1, 1):
+            raise ValueError("groups of experts come with softmax_all scores")
+        if not 0 < self.groups[1] <= self.groups[0] or self.routed % self.groups[0] or self.top > self.groups[1] * (self.routed // self.groups[0]):
+            raise ValueError(f"{self.top} of {self.routed} experts cannot be chosen from {self.groups[1]} of {self.groups[0]} groups")
         if not self.limit > 0:
             raise ValueError(f"the experts' limit must be positive, got {self.limit}")
         self.shared = build_part(p["shared"], self.join(prefix, "shared")) if p.get("shared") is not None else None
+        self.correction = None
         self.w_router = self.b_router = self.w_gate = self.w_up = self.w_down = None
 
     def parts(self):
@@ -87,9 +104,12 @@ class RoutedExperts(FeedForward):
         if p.get("router", "linear") == "table":
             out.append(WeightSpec(f"{prefix}.table", (int(p["vocab_size"]), int(p["top"])), kind="int", init="distinct", free=e))
         else:
-            out.append(WeightSpec(f"{prefix}.router", (e, h)))
+            routed = e + int(p.get("identity") or 0)
+            out.append(WeightSpec(f"{prefix}.router", (routed, h)))
             if p.get("router_bias", True) is not False:
-                out.append(WeightSpec(f"{prefix}.router.b", (e,), kind="vector"))
+                out.append(WeightSpec(f"{prefix}.router.b", (routed,), kind="vector"))
+            if p.get("score") == "softmax_all":
+                out.append(WeightSpec(f"{prefix}.correction", (routed,), kind="vector"))
         if p.get("shared") is not None:
             out += part_class(p["shared"].kind).weight_specs(p["shared"], cls.join(prefix, "shared"))
         return out
@@ -113,6 +133,8 @@ class RoutedExperts(FeedForward):
         else:
             self.w_router = rt.matrix(weights.get(f"{self.prefix}.router"))
             self.b_router = rt.vector(weights.get(f"{self.prefix}.router.b")) if self.router_bias else None
+            if self.score == "softmax_all":
+                self.correction = rt.vector(weights.get(f"{self.prefix}.correction"))
             rt.kernels.experts_lib()
         if not self.tabled and self.top > rt.kernels.experts_max_top():
             raise ValueError(f"{self.top} experts a token exceed the {rt.kernels.experts_max_top()} the routing kernel picks")
@@ -130,7 +152,7 @@ class RoutedExperts(FeedForward):
         ``"any"`` in every step (a reader that takes slices of any number of rows)."""
         rt = ctx.rt
         k = rt.kernels
-        t, e, top = ctx.n_tokens, self.experts, self.top
+        t, e, top = ctx.n_tokens, self.routed, self.top
         rows = self.rows_a_tile(t, top, e)
         cap = k.experts_tile_capacity(t, e, top, rows)
         chosen = ctx.buf("experts.chosen", (t * top,), torch.int32)
@@ -143,12 +165,13 @@ class RoutedExperts(FeedForward):
         else:
             logits = ctx.buf("experts.logits", (t, e), torch.float32)
             k.gemm(x, self.w_router, logits, STORE_F32)
-            k.experts_route(logits, self.b_router, top, rows, chosen, share, order, tiles, counts, scoring=self.score)
+            k.experts_route(logits, self.b_router, top, rows, chosen, share, order, tiles, counts, scoring=self.score,
+                            correction=self.correction, groups=self.groups)
         slices = top + (1 if self.shared is not None else 0)
         partials = ctx.buf("experts.slices", (slices * t, self.hidden), torch.float32).view(slices, t, self.hidden)
         act = ctx.buf("experts.act", (t * top, self.inter), rt.dtype)
         k.experts_apply(x, self.w_gate, self.w_up, self.w_down, top, rows, order, tiles, share, self.limit, self.alpha,
-                        act, partials[:top], shift=self.shift, weigh_input=self.weigh == "input")
+                        act, partials[:top], shift=self.shift, weigh_input=self.weigh == "input", identity=self.identity)
         if self.shared is not None:
             self.shared.forward(ctx, x, partials[top], accumulate=False)
         pending = PendingAdd(partials)

@@ -8,6 +8,17 @@ from ..config.base import PartSpec
 from .base import Norm, WeightSpec, register_part
 
 
+def sum_of_copies(ctx, x, norm, pending, out, rows) -> None:
+    """``norm`` (a part with ``step_norm``) of the sum of the stream's copies, after what the last sublayer still has to
+    write into them."""
+    if pending is not None and not hasattr(pending, "mix"):
+        raise ValueError("a stream of several copies takes the pending write of its own arrangement only")
+    weight, eps, centred, bias = (tuple(norm.step_norm()) + (None,))[:4]
+    ctx.rt.kernels.streams_step(x, norm.copies, None if pending is None else pending.partials,
+                                None if pending is None else pending.mix, None if pending is None else pending.gain,
+                                None, weight, eps, out, rows, bias=bias, centred=centred)
+
+
 @register_part("rmsnorm")
 class RMSNorm(Norm):
     """Parameters: ``size``, ``eps``; ``name`` overrides the tensor name.  With ``optional`` the
@@ -53,12 +64,7 @@ class RMSNorm(Norm):
             pending.step(ctx, x, self.step_norm(), out, rows)
             return
         if self.copies > 1 or hasattr(pending, "mix"):
-            # the sum of the copies, after what the last sublayer still has to write into them
-            if pending is not None and not hasattr(pending, "mix"):
-                raise ValueError("a stream of several copies takes the pending write of its own arrangement only")
-            ctx.rt.kernels.streams_step(x, self.copies, None if pending is None else pending.partials,
-                                        None if pending is None else pending.mix, None if pending is None else pending.gain,
-                                        None, self.weight, self.eps, out, rows)
+            sum_of_copies(ctx, x, self, pending, out, rows)
             return
         if pending is not None:
             ctx.rt.kernels.add_rmsnorm(x, pending.partials, self.weight, out, self.eps, rows)
@@ -73,9 +79,10 @@ class RMSNorm(Norm):
 
 @register_part("layernorm")
 class LayerNorm(Norm):
-    """``y = (x - mean) / sqrt(mean((x - mean)^2) + eps) * w`` in 32-bit, no bias.  Parameters: ``size``, ``eps``; ``name``
-    overrides the tensor name (default: the prefix itself).  With ``optional`` the weight may be absent (a layer whose
-    second half is missing never runs the norm)."""
+    """``y = (x - mean) / sqrt(mean((x - mean)^2) + eps) * w (+ b)`` in 32-bit.  Parameters: ``size``, ``eps``; ``name``
+    overrides the tensor name (default: the prefix itself); ``bias`` (default False: no bias): the tensor ``<name>.b``.
+    With ``optional`` the tensors may be absent (a layer whose second half is missing never runs the norm).  ``copies``
+    (default 1): the stream holds that many copies ``[T, copies * size]`` and the norm reads their sum."""
 
     graph_safe = True
     repeatable = True
@@ -84,7 +91,8 @@ class LayerNorm(Norm):
         super().__init__(spec, prefix)
         self.size = int(spec["size"])
         self.eps = float(spec["eps"])
-        self.weight = None
+        self.copies = int(spec.params.get("copies") or 1)
+        self.weight = self.bias = None
 
     @staticmethod
     def tensor_name(spec: PartSpec, prefix: str) -> str:
@@ -92,24 +100,30 @@ class LayerNorm(Norm):
 
     @classmethod
     def weight_specs(cls, spec: PartSpec, prefix: str) -> list[WeightSpec]:
-        return [WeightSpec(cls.tensor_name(spec, prefix), (int(spec["size"]),), kind="vector", init="norm",
-                           optional=bool(spec.params.get("optional")))]
+        name, size, optional = cls.tensor_name(spec, prefix), int(spec["size"]), bool(spec.params.get("optional"))
+        out = [WeightSpec(name, (size,), kind="vector", init="norm", optional=optional)]
+        if spec.params.get("bias"):
+            out.append(WeightSpec(f"{name}.b", (size,), kind="vector", optional=optional))
+        return out
 
     def load(self, weights, rt) -> None:
         name = self.tensor_name(self.spec, self.prefix)
         if self.spec.params.get("optional") and name not in weights:
             return
         self.weight = rt.vector(weights.get(name))
+        if self.spec.params.get("bias"):
+            self.bias = rt.vector(weights.get(f"{name}.b"))
         rt.kernels.mixers_lib()
 
     def step_norm(self):
-        """The norm as ``Kernels.residual_step`` takes it: (weight, eps, whether the mean is subtracted)."""
-        return self.weight, self.eps, True
+        """The norm as ``Kernels.residual_step`` takes it: (weight, eps, whether the mean is subtracted, bias)."""
+        return self.weight, self.eps, True, self.bias
 
     def forward(self, ctx, x, out, rows=None, pending=None) -> None:
         """``pending`` (a ``PendingAdd``): added to ``x`` first, in the same launch."""
-        if hasattr(pending, "mix"):
-            raise ValueError("layernorm does not read a residual stream of several copies")
+        if self.copies > 1 or hasattr(pending, "mix"):
+            sum_of_copies(ctx, x, self, pending, out, rows)
+            return
         if hasattr(pending, "post"):
             pending.step(ctx, x, self.step_norm(), out, rows)
             return

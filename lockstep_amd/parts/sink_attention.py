@@ -32,7 +32,7 @@ import torch
 
 from ..config.base import PartSpec
 from ..ops import STORE_F32
-from .base import Mixer, PagedKVSpec, WeightSpec, build_part, project_out, register_part
+from .base import PagedKVSpec, ProjectedMixer, WeightSpec, build_part, project_out, register_part, stack_rows
 
 TILE_KEYS = 32         # keys of a tile of the attention kernel
 MAX_RUNS = 16          # the most runs the keys of a row block are dealt to
@@ -59,14 +59,15 @@ def distance_buckets(rows: int, farthest: float) -> list[int]:
 
 
 @register_part("sink_attention")
-class SinkAttention(Mixer):
+class SinkAttention(ProjectedMixer):
     """Parameters: ``hidden_size``, ``num_heads``, ``num_kv_heads``, ``head_dim`` (queries and keys),
     ``value_dim``, ``position`` (a position-encoding ``PartSpec``), ``scale``, ``window`` / ``chunk``
     (None or a size; at most one of them), ``keep_first`` (with a window: the first that many tokens stay visible), ``sink`` (None, ``"zero"`` or ``"learned"``), ``gate``,
     ``bias`` (biases of q, k, v), ``out_bias``, ``qk_norm`` (None or the eps of a norm over the whole
     projection), ``head_norm`` (None or the eps of a norm over every head of q and of k; without weights, or with ``head_norm_weights`` times
     ``q.norm`` / ``k.norm`` of ``head_dim`` elements that all heads share), ``shared_kv`` (the values are the keys as projected), ``distance_bias`` (None or
-    ``{"farthest": D, "rows": B}``; ``rows`` only sizes random weights, a checkpoint's table says it itself).
+    ``{"farthest": D, "rows": B}``; ``rows`` only sizes random weights, a checkpoint's table says it itself),
+    ``out_scale`` (default 1; the values are stored times it).
     Tensors below the prefix: ``q``, ``k``, ``v``, ``o``; ``g`` (gate); ``q.b``, ``k.b``, ``v.b``;
     ``o.b``; ``q.norm``, ``k.norm``; ``rel [B, H]``; ``sink [H]``."""
 
@@ -98,6 +99,8 @@ class SinkAttention(Mixer):
             raise ValueError(f"keep_first {self.keep_first} must not be negative and needs a window")
         self.shared_kv = bool(p.get("shared_kv"))
         self.distance_bias = p.get("distance_bias")
+        self.out_scale = 1.0 if p.get("out_scale") is None else float(p["out_scale"])
+        self.out_width = self.nq * self.dv
         if self.nq % self.nkv:
             raise ValueError(f"{self.nq} query heads are not a multiple of {self.nkv} kv heads")
         if self.window < 0 or self.chunk < 0 or (self.window and self.chunk):
@@ -150,13 +153,19 @@ class SinkAttention(Mixer):
         return PagedKVSpec(self.nkv, self.dk, self.window or None, value_dim=self.dv, chunk=self.chunk or None,
                            keep_first=self.keep_first)
 
-    def load(self, weights, rt) -> None:
+    def in_matrices(self, weights) -> list:
         names = ["q", "k"] + ([] if self.shared_kv else ["v"]) + (["g"] if self.gate else [])
-        mats = [weights.get(f"{self.prefix}.{n}") for n in names]
-        if len({m.dtype for m in mats}) > 1:
-            mats = [m.to(torch.float32) for m in mats]
-        self.w_in = rt.matrix(torch.cat(mats, dim=0))
-        self.w_o = rt.matrix(weights.get(f"{self.prefix}.o"))
+        return [weights.get(f"{self.prefix}.{n}") for n in names]
+
+    def out_matrix(self, weights):
+        return weights.get(f"{self.prefix}.o")
+
+    def load(self, weights, rt) -> None:
+        self.w_in = rt.matrix(stack_rows(self.in_matrices(weights)))
+        self.w_o = rt.matrix(self.out_matrix(weights))
+        self.load_own(weights, rt)
+
+    def load_own(self, weights, rt) -> None:
         if self.bias:
             biased = ["q", "k"] + ([] if self.shared_kv else ["v"])
             self.b_in = rt.vector(torch.cat([weights.get(f"{self.prefix}.{n}.b").to(torch.float32) for n in biased]))
@@ -277,24 +286,20 @@ class SinkAttention(Mixer):
         ctx.declare(key, ints, signature=("sink_attention", len(items), n_folds, row_tiles))
         ctx.notes[key] = (len(items), n_folds, row_tiles)
 
-    def forward(self, ctx, run, x, out, accumulate: bool, defer: bool = False):
-        rt = ctx.rt
-        k = rt.kernels
+    def mix(self, ctx, run, raw, out) -> None:
+        k = ctx.rt.kernels
         t = ctx.n_tokens
         nq, nkv, d, dv = self.nq, self.nkv, self.d, self.dv
         group, key_pages, value_pages = ctx.cache.unit_pages(run.cache)
         if not run.writes_cache:
             raise ValueError("a sink attention layer writes its own keys and values")
-        raw = ctx.buf("sink.in_f32", (t, self.w_in.shape[0]), torch.float32)
-        k.gemm(x, self.w_in, raw, STORE_F32)
-        q = ctx.buf("sink.q", (t, nq * self.dk), rt.dtype)
+        q = ctx.buf("sink.q", (t, nq * self.dk), ctx.rt.dtype)
         k.qkv_post(raw, t, nq, nkv, d, dv, self.b_in, self.q_norm, self.k_norm, self.qk_norm or self.head_norm or 0.0, self.position.cos,
                    self.position.sin, self.position.rotary_dim, self.neighbours, ctx.max_position, ctx.tok_seq,
                    ctx.tok_pos, ctx.seqs, group.table, q, key_pages, value_pages, group.page_size,
                    keys_are_values=self.shared_kv, key_pad=self.dk, per_head=self.head_norm is not None,
-                   head_weights=self.head_norm_weights)
+                   head_weights=self.head_norm_weights, value_scale=self.out_scale)
         key = self._block_key()
-        attn = ctx.buf("sink.out", (t, nq * dv), rt.dtype)
         n_items, n_folds, row_tiles = ctx.notes[key]
         work = ctx.block(key)
         part_rows = k.sink_staged_rows(nq, nkv) if row_tiles == STAGED else 16 * row_tiles if row_tiles else 1
@@ -302,8 +307,15 @@ class SinkAttention(Mixer):
         gate = raw[:, raw.shape[1] - nq * dv:] if self.gate else None
         k.sink_attention(q, nq, nkv, self.dk, dv, key_pages, value_pages, group.page_size, group.table, ctx.seqs,
                          work[:4 * n_items], n_items, row_tiles, self.scale, self.window, self.chunk, self.sink,
-                         self.by_distance, gate, attn, work[4 * n_items:] if n_folds else None, n_folds, part,
+                         self.by_distance, gate, out, work[4 * n_items:] if n_folds else None, n_folds, part,
                          keep_first=self.keep_first)
+
+    def forward(self, ctx, run, x, out, accumulate: bool, defer: bool = False):
+        k = ctx.rt.kernels
+        raw = ctx.buf("sink.in_f32", (ctx.n_tokens, self.w_in.shape[0]), torch.float32)
+        k.gemm(x, self.w_in, raw, STORE_F32)
+        attn = ctx.buf("sink.out", (ctx.n_tokens, self.out_width), ctx.rt.dtype)
+        self.mix(ctx, run, raw, attn)
         if self.b_o is not None:
             # (a product with an output bias is added to the stream at once, then the bias: the same order
             # of additions at every batch size)
