@@ -43,8 +43,9 @@ the Narurax design (an embedding that adds a table of token pairs, mixer inputs 
 delta rule with a decay a channel, attention whose weights are mixed over the heads, attention with a norm a head,
 windows that keep the first tokens, experts with sigmoid scores on their input) or, with ``--designs
 qwen3,toripel,tukavik``, the Tukavik design (norms on both sides of every sublayer, averages over depth, a recurrence of one
-number a channel, attention over a cached latent without positions, two-matrix feed-forwards with xIELU; ``--designs``
-chooses) beside the Qwen3 decoder at the same layer sizes (width, feed-forward, heads, head size, layers, vocabulary), both
+number a channel, attention over a cached latent without positions, two-matrix feed-forwards with xIELU) or, with ``--designs
+qwen3,toripel,pozozen``, the Pozozen design (a residual stream of four copies under layer norms, attention and a state-space
+recurrence side by side, a matrix memory with exponential gates, experts in groups with a shared one; ``--designs`` chooses) beside the Qwen3 decoder at the same layer sizes (width, feed-forward, heads, head size, layers, vocabulary), both
 with random weights: prefill of one prompt and decode steps at batch 1 and 8, each with its
 fraction of the roofline.
 """
@@ -471,6 +472,26 @@ def tukavik_like(qwen, layers: int):
                              "norm": {"eps": qwen.rms_norm_eps}, "layers": out})
 
 
+def pozozen_like(qwen, layers: int, window: int = 4096, experts: int = 32, top: int = 4, streams: int = 4):
+    """A Pozozen configuration at the layer sizes of the Qwen3 configuration ``qwen``: a residual stream of four copies; the
+    layers alternate between windowed attention beside a state-space recurrence and the matrix memory; every mixer has the heads
+    and head size of the Qwen3 attention (the state-space one: states of ``head_dim`` rows, one group, four taps).  A token's
+    feed-forward multiplies with as many weights as the dense one: a shared expert of half its size and ``top`` routed ones of
+    ``1 / (2 top)`` each, of four groups of which two are kept; one expert in nine returns its input instead."""
+    from lockstep_amd.config import config_from_dict
+
+    heads, kv, d = qwen.num_attention_heads, qwen.num_key_value_heads, qwen.head_dim
+    moe = {"kind": "moe", "expert": {"ff": qwen.intermediate_size // (2 * top)}, "shared": {"ff": qwen.intermediate_size // 2},
+           "router": {"experts": experts, "identity": experts // 8, "top": top, "groups": {"count": 4, "keep": 2}}}
+    both = {"left": {"heads": heads, "kv_heads": kv, "dim": d, "vdim": d, "scale": d ** -0.5, "mask": {"size": window}}, "left_scale": 0.5,
+            "right": {"heads": heads, "vdim": d, "state": d, "groups": 1, "conv": 4, "norm_groups": 1}, "right_scale": 0.5}
+    memory = {"heads": heads, "dim": d, "vdim": d, "gate_cap": 15.0}
+    cycle = [{"type": "parallel", "mixer": both, "mlp": moe}, {"type": "mlstm", "mixer": memory, "mlp": moe}]
+    return config_from_dict({"architecture": "Pozozen", "vocab": qwen.vocab_size, "width": qwen.hidden_size,
+                             "norm": {"eps": qwen.rms_norm_eps}, "residual_mult": 0.5, "streams": streams,
+                             "layers": [cycle[i % 2] for i in range(layers)]})
+
+
 def designs_record(args) -> dict:
     """Prefill and decode of the other designs beside Qwen3 at equal layer sizes."""
     import gc
@@ -490,7 +511,7 @@ def designs_record(args) -> dict:
            "data": "synthetic: uniform random token ids, random weights", "designs": {}}
     makers = {"qwen3": lambda: qwen, "bikovik": lambda: bikovik_like(qwen, layers), "biberax": lambda: biberax_like(qwen, layers),
               "toripel": lambda: toripel_like(qwen, layers), "narurax": lambda: narurax_like(qwen, layers),
-              "tukavik": lambda: tukavik_like(qwen, layers)}
+              "tukavik": lambda: tukavik_like(qwen, layers), "pozozen": lambda: pozozen_like(qwen, layers)}
     for name in args.designs.split(","):
         if name not in makers:
             raise SystemExit(f"--designs: {name!r} is not one of {', '.join(makers)}")
@@ -670,7 +691,7 @@ def main(argv=None) -> int:
                         "scheduler; contexts: prefill and decode at the context lengths of --contexts; designs: "
                         "the Bikovik and Biberax designs beside Qwen3 at the layer sizes of --model")
     p.add_argument("--contexts", default="4096,8192,16384", help="contexts: the context lengths, comma separated")
-    p.add_argument("--designs", default="qwen3,bikovik,biberax", help="designs: which of qwen3, bikovik, biberax, toripel, narurax, tukavik, comma separated")
+    p.add_argument("--designs", default="qwen3,bikovik,biberax", help="designs: which of qwen3, bikovik, biberax, toripel, narurax, tukavik, pozozen, comma separated")
     p.add_argument("--repeats", type=int, default=5, help="timed runs; the median is reported with the spread")
     p.add_argument("--requests", type=int, default=0, help="serve: only the first N requests of the workload")
     p.add_argument("--prefill-chunk", type=int, default=None, help="serve: prompt portion (0: whole prompts)")

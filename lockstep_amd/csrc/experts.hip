@@ -50,11 +50,26 @@ struct Choice {
   const float* correction;   // [E], scoring 2
 };
 
+// A lane's (value, index) against those of the lane that a data-parallel move inside its row of sixteen names; the larger
+// value stays, the lower index winning a tie (0x7fffffff: none).
+__device__ __forceinline__ void keep_better(float& v, int& e, float ov, int oe) {
+  const bool take = oe != 0x7fffffff && (e == 0x7fffffff || ov > v || (ov == v && oe < e));
+  v = take ? ov : v;
+  e = take ? oe : e;
+}
+template <int CTRL>
+__device__ __forceinline__ void keep_better_of(float& v, int& e) {
+  keep_better(v, e, __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), CTRL, 0xF, 0xF, true)),
+              __builtin_amdgcn_mov_dpp(e, CTRL, 0xF, 0xF, true));
+}
+
+// PL: experts a lane holds
+template <int PL>
 __device__ __forceinline__ void pick_top(const float* __restrict__ row, const float* __restrict__ bias, int E, int top,
                                          int lane, int* __restrict__ picked, float* __restrict__ share, const Choice& how) {
-  float mine[kMaxPerLane], score[kMaxPerLane];
+  float mine[PL], score[PL];
 #pragma unroll
-  for (int m = 0; m < kMaxPerLane; ++m) {
+  for (int m = 0; m < PL; ++m) {
     const int e = lane + 64 * m;
     mine[m] = e < E ? row[e] + (bias ? bias[e] : 0.f) : 0.f;
     score[m] = 0.f;
@@ -64,21 +79,21 @@ __device__ __forceinline__ void pick_top(const float* __restrict__ row, const fl
     best_v = 0.f;
     best = 0x7fffffff;
 #pragma unroll
-    for (int m = 0; m < kMaxPerLane; ++m) {
+    for (int m = 0; m < PL; ++m) {
       const int e = lane + 64 * m;
       if (e < E && !((closed >> m) & 1u) && (best == 0x7fffffff || mine[m] > best_v)) {
         best_v = mine[m];
         best = e;
       }
     }
+    // pairs, pairs of pairs, the mirror image of the half row and of the row (after each, the lanes that met agree), then
+    // the rows of sixteen
+    keep_better_of<0xB1>(best_v, best);
+    keep_better_of<0x4E>(best_v, best);
+    keep_better_of<0x141>(best_v, best);
+    keep_better_of<0x140>(best_v, best);
 #pragma unroll
-    for (int step = 1; step < 64; step <<= 1) {
-      const float other_v = __shfl_xor(best_v, step, kWave);
-      const int other = __shfl_xor(best, step, kWave);
-      const bool take = other != 0x7fffffff && (best == 0x7fffffff || other_v > best_v || (other_v == best_v && other < best));
-      best_v = take ? other_v : best_v;
-      best = take ? other : best;
-    }
+    for (int step = 16; step < 64; step <<= 1) keep_better(best_v, best, __shfl_xor(best_v, step, kWave), __shfl_xor(best, step, kWave));
   };
   unsigned taken = 0;
   if (how.scoring == 2) {
@@ -87,13 +102,13 @@ __device__ __forceinline__ void pick_top(const float* __restrict__ row, const fl
     largest(0u, top_z, at);
     float part = 0.f;
 #pragma unroll
-    for (int m = 0; m < kMaxPerLane; ++m) {
+    for (int m = 0; m < PL; ++m) {
       score[m] = lane + 64 * m < E ? expf(mine[m] - top_z) : 0.f;
       part = part + score[m];
     }
     const float inv = 1.0f / wave_sum(part);
 #pragma unroll
-    for (int m = 0; m < kMaxPerLane; ++m) {
+    for (int m = 0; m < PL; ++m) {
       score[m] = score[m] * inv;
       if (lane + 64 * m < E) mine[m] = score[m] + how.correction[lane + 64 * m];
     }
@@ -105,7 +120,7 @@ __device__ __forceinline__ void pick_top(const float* __restrict__ row, const fl
         int best;
         largest(open, v, best);
 #pragma unroll
-        for (int m = 0; m < kMaxPerLane; ++m)
+        for (int m = 0; m < PL; ++m)
           if ((lane + 64 * m) / each == best / each) open |= 1u << m;
       }
       taken = ~open;
@@ -122,7 +137,7 @@ __device__ __forceinline__ void pick_top(const float* __restrict__ row, const fl
     if (how.scoring == 2) {   // (the weight is the score without the correction)
       float held = 0.f;
 #pragma unroll
-      for (int m = 0; m < kMaxPerLane; ++m) held = (best >> 6) == m ? score[m] : held;
+      for (int m = 0; m < PL; ++m) held = (best >> 6) == m ? score[m] : held;
       best_v = __shfl(held, best & 63, kWave);
     }
     if (lane == k) {
@@ -157,12 +172,13 @@ __global__ __launch_bounds__(256) void route_table_kernel(const int* __restrict_
   weight[pair] = 1.0f / (float)top;
 }
 
+template <int PL>
 __global__ __launch_bounds__(256) void route_topk_kernel(const float* __restrict__ z, long ldz,
                                                          const float* __restrict__ bias, int n_tokens, int E, int top,
                                                          int* __restrict__ expert, float* __restrict__ weight, Choice how) {
   const int t = blockIdx.x * 4 + (threadIdx.x >> 6);
   if (t >= n_tokens) return;
-  pick_top(z + (long)t * ldz, bias, E, top, threadIdx.x & 63, expert + (long)t * top, weight + (long)t * top, how);
+  pick_top<PL>(z + (long)t * ldz, bias, E, top, threadIdx.x & 63, expert + (long)t * top, weight + (long)t * top, how);
 }
 
 // ---------------------------------------------------------------------------
@@ -241,6 +257,7 @@ __global__ __launch_bounds__(64) void route_place_kernel(const int* __restrict__
 
 constexpr int kSmallPairs = 512, kSmallExperts = 512;   // what the one-workgroup kernel keeps in LDS
 
+template <int PL>
 __global__ __launch_bounds__(1024) void route_small_kernel(const float* __restrict__ z, long ldz,
                                                            const float* __restrict__ bias, int n_tokens, int E, int top,
                                                            int rows_a_tile, int* __restrict__ expert,
@@ -262,7 +279,7 @@ __global__ __launch_bounds__(1024) void route_small_kernel(const float* __restri
     }
   }
   for (int t = w; t < n_tokens && !table; t += 16) {
-    pick_top(z + (long)t * ldz, bias, E, top, lane, picks_s + t * top, share_s[w], how);
+    pick_top<PL>(z + (long)t * ldz, bias, E, top, lane, picks_s + t * top, share_s[w], how);
     if (lane < top) {
       expert[(long)t * top + lane] = picks_s[t * top + lane];
       weight[(long)t * top + lane] = share_s[w][lane];
@@ -672,12 +689,18 @@ extern "C" int ls_experts_route(const float* z, long ldz, const float* bias, int
   LS_REQUIRE(E <= 64 * kMaxPerLane, "experts_route: %d experts, the routing kernel takes %d", E, 64 * kMaxPerLane);
   hipStream_t s = reinterpret_cast<hipStream_t>(stream);
   const int P = n_tokens * top;
-  if (P <= kSmallPairs && E <= kSmallExperts) {
-    hipLaunchKernelGGL(route_small_kernel, dim3(1), dim3(1024), 0, s, z, ldz, bias, n_tokens, E, top, rows_a_tile,
-                       expert, weight, order, tiles, cap, (const int*)nullptr, (const int*)nullptr, how);
-  } else {
-    hipLaunchKernelGGL(route_topk_kernel, dim3((n_tokens + 3) / 4), dim3(256), 0, s, z, ldz, bias, n_tokens, E, top,
+#define LS_ROUTE(PL_)                                                                                                     \
+  if (P <= kSmallPairs && E <= kSmallExperts)                                                                             \
+    hipLaunchKernelGGL(route_small_kernel<PL_>, dim3(1), dim3(1024), 0, s, z, ldz, bias, n_tokens, E, top, rows_a_tile,   \
+                       expert, weight, order, tiles, cap, (const int*)nullptr, (const int*)nullptr, how);                 \
+  else                                                                                                                    \
+    hipLaunchKernelGGL(route_topk_kernel<PL_>, dim3((n_tokens + 3) / 4), dim3(256), 0, s, z, ldz, bias, n_tokens, E, top, \
                        expert, weight, how);
+  if (E <= 64) { LS_ROUTE(1) }
+  else if (E <= 128) { LS_ROUTE(2) }
+  else { LS_ROUTE(kMaxPerLane) }
+#undef LS_ROUTE
+  if (!(P <= kSmallPairs && E <= kSmallExperts)) {
     hipLaunchKernelGGL(route_count_kernel, dim3(E), dim3(64), 0, s, expert, P, counts);
     hipLaunchKernelGGL(route_place_kernel, dim3(E), dim3(64), 0, s, expert, counts, P, E, rows_a_tile, order, tiles, cap);
   }
@@ -695,7 +718,7 @@ extern "C" int ls_experts_route_table(const int* token_ids, const int* table, in
   hipStream_t s = reinterpret_cast<hipStream_t>(stream);
   const int P = n_tokens * top;
   if (P <= kSmallPairs && E <= kSmallExperts) {
-    hipLaunchKernelGGL(route_small_kernel, dim3(1), dim3(1024), 0, s, (const float*)nullptr, 0L, (const float*)nullptr,
+    hipLaunchKernelGGL(route_small_kernel<1>, dim3(1), dim3(1024), 0, s, (const float*)nullptr, 0L, (const float*)nullptr,
                        n_tokens, E, top, rows_a_tile, expert, weight, order, tiles, cap, token_ids, table, Choice{0, 1, 1, nullptr});
   } else {
     hipLaunchKernelGGL(route_table_kernel, dim3((P + 255) / 256), dim3(256), 0, s, token_ids, table, n_tokens, top, expert,

@@ -173,32 +173,46 @@ __global__ __launch_bounds__(64) void exp_gates_kernel(const float* __restrict__
   float* kept = state + (long)m.table_row * state_stride + m_at + 2 * h;
   float front = kept[m.q_start & 1];
   const float bi = i_bias[h], bf = f_bias[h];
-  for (int t0 = 0; t0 < m.q_len; t0 += 64) {
-    const bool in = t0 + lane < m.q_len;
+  constexpr int AHEAD = 4;   // blocks of 64 tokens whose logits are on their way
+  float zi[AHEAD], zf[AHEAD];
+  auto request = [&](int t0, float& i, float& f) LS_INLINED {
     const float* row = raw + (long)(m.q_off + min(t0 + lane, m.q_len - 1)) * ld;
-    float i, f;
-    exp_gate_values(row[i_at + h] + bi, row[f_at + h] + bf, cap, i, f);
-    float F = in ? f : 0.f, M = in ? i : -3e38f;   // m behind this run of tokens: max(F + m in front, M)
+    i = row[i_at + h];
+    f = row[f_at + h];
+  };
 #pragma unroll
-    for (int step = 1; step < 64; step <<= 1) {
-      const float oF = __shfl_up(F, step, kWave), oM = __shfl_up(M, step, kWave);
-      if (lane >= step) {
-        M = fmaxf(F + oM, M);
-        F = F + oF;
+  for (int u = 0; u < AHEAD; ++u) request(64 * u, zi[u], zf[u]);
+  for (int tb = 0; tb < m.q_len; tb += 64 * AHEAD) {
+#pragma unroll
+    for (int u = 0; u < AHEAD; ++u) {
+      const int t0 = tb + 64 * u;
+      if (t0 >= m.q_len) break;
+      const bool in = t0 + lane < m.q_len;
+      float i, f;
+      exp_gate_values(zi[u] + bi, zf[u] + bf, cap, i, f);
+      request(t0 + 64 * AHEAD, zi[u], zf[u]);
+      float F = in ? f : 0.f, M = in ? i : -3e38f;   // m behind this run of tokens: max(F + m in front, M)
+#pragma unroll
+      for (int step = 1; step < 64; step <<= 1) {
+        const float oF = __shfl_up(F, step, kWave), oM = __shfl_up(M, step, kWave);
+        if (lane >= step) {
+          M = fmaxf(F + oM, M);
+          F = F + oF;
+        }
       }
+      const float mine = fmaxf(F + front, M);
+      float before = __shfl_up(mine, 1, kWave);
+      if (lane == 0) before = front;
+      if (in) {
+        Gate g;
+        g.la = fminf(f + before - mine, 0.f);
+        g.b = expf(i - mine);
+        g.floor = expf(-mine);
+        g.nq = 0.f;
+        gates[(long)(m.q_off + t0 + lane) * H + h] = g;
+      }
+      front = __shfl(mine, 63, kWave);   // (lanes beyond the last token repeat its maximum: F and M are the identity there)
     }
-    const float mine = fmaxf(F + front, M);
-    float before = __shfl_up(mine, 1, kWave);
-    if (lane == 0) before = front;
-    if (in) {
-      Gate g;
-      g.la = fminf(f + before - mine, 0.f);
-      g.b = expf(i - mine);
-      g.floor = expf(-mine);
-      g.nq = 0.f;
-      gates[(long)(m.q_off + t0 + lane) * H + h] = g;
-    }
-    front = __shfl(mine, 63, kWave);   // (lanes beyond the last token repeat its maximum: F and M are the identity there)
   }
   if (lane == 0) kept[m.kv_len & 1] = front;
 }
@@ -370,6 +384,7 @@ __global__ __launch_bounds__(256) void memory_token_kernel(const float* __restri
     const int each = H / sp.G, g = h / each, inner = H * DV;
     const bool writes_group = cb == 0 && h == g * each;
     float* ring = slot + sp.ring_at;
+    const int own_row = pos % sp.M, first_row = own_row + 1;   // (position pos - (M-1) + j lies in row (pos + 1 + j) mod M)
     for (int i = threadIdx.x; i < 2 * N + kMemCols; i += 256) {
       const bool is_v = i >= 2 * N;
       const int vc = cb * kMemCols + i - 2 * N;
@@ -380,13 +395,25 @@ __global__ __launch_bounds__(256) void memory_token_kernel(const float* __restri
       const int c = is_v ? h * DV + vc : (i < N ? inner + g * N + i : inner + sp.G * N + g * N + (i - N));
       const float now = row[sp.x_at + c];
       float y = sp.conv_bias[c];
-      for (int j = 0; j + 1 < sp.M; ++j)   // inputs at the positions pos - (M-1) + j: rows of the ring (zeros before the start)
-        y = y + sp.taps[(long)j * sp.C + c] * ring[(long)((pos + 1 + j) % sp.M) * sp.C + c];
+      // inputs at the positions pos - (M-1) + j: rows of the ring (zeros before the start), requested together four at a time
+      for (int j0 = 0; j0 + 1 < sp.M; j0 += 4) {
+        float tap[4], in[4];
+#pragma unroll
+        for (int u = 0; u < 4; ++u) {
+          const int j = min(j0 + u, sp.M - 2);
+          const int r = first_row + j;
+          tap[u] = sp.taps[(long)j * sp.C + c];
+          in[u] = ring[(long)(r >= sp.M ? r - sp.M : r) * sp.C + c];
+        }
+#pragma unroll
+        for (int u = 0; u < 4; ++u)
+          if (j0 + u + 1 < sp.M) y = y + tap[u] * in[u];
+      }
       y = silu_m(y + sp.taps[(long)(sp.M - 1) * sp.C + c] * now);
       if (is_v) v_s[i - 2 * N] = y;
       else if (i < N) k_s[i] = y;
       else q_s[i - N] = y;
-      if (is_v || writes_group) ring[(long)(pos % sp.M) * sp.C + c] = now;
+      if (is_v || writes_group) ring[(long)own_row * sp.C + c] = now;
     }
     const float dt = softplus_m(row[sp.dt_at + h] + sp.dt_bias[h]);
     a = expf(-expf(sp.a_log[h]) * dt);
@@ -703,9 +730,8 @@ __global__ __launch_bounds__(256) void memory_chunk_out_kernel(HeadRows q, HeadR
 // runs of neighbours (eps inside the root), times weight [inner]; stored as T.  A workgroup a (token, part): thread t
 // adds the squares of the elements t, t + 256, ... ascending, then a butterfly over the wave and the waves in order.
 // ---------------------------------------------------------------------------
-constexpr int kGatedPer = 16;   // gated elements a thread keeps between the sum and the scaling (more are formed again)
-
-template <typename T>
+// (PER: gated elements a thread keeps between the sum and the scaling; those of longer parts are formed again)
+template <typename T, int PER>
 __global__ __launch_bounds__(256) void gated_parts_norm_kernel(const float* __restrict__ y, long ldy, const float* __restrict__ z,
                                                                long ldz, int each, const float* __restrict__ weight, float eps,
                                                                T* __restrict__ out, long ldo) {
@@ -714,16 +740,20 @@ __global__ __launch_bounds__(256) void gated_parts_norm_kernel(const float* __re
   const int at = blockIdx.y * each;
   const float* y_row = y + t * ldy + at;
   const float* z_row = z + t * ldz + at;
-  float mine[kGatedPer];
+  float mine[PER], gate[PER];
   float part = 0.f;
 #pragma unroll
-  for (int j = 0; j < kGatedPer; ++j) {
+  for (int j = 0; j < PER; ++j) {   // (addresses that are always valid: no branch between the loads)
     const int c = threadIdx.x + 256 * j;
-    mine[j] = c < each ? y_row[c] * silu_m(z_row[c]) : 0.f;
+    mine[j] = y_row[c < each ? c : 0];
+    gate[j] = z_row[c < each ? c : 0];
   }
 #pragma unroll
-  for (int j = 0; j < kGatedPer; ++j) part = part + mine[j] * mine[j];
-  for (int c = threadIdx.x + 256 * kGatedPer; c < each; c += 256) {
+  for (int j = 0; j < PER; ++j) {
+    mine[j] = (int)threadIdx.x + 256 * j < each ? mine[j] * silu_m(gate[j]) : 0.f;
+    part = part + mine[j] * mine[j];
+  }
+  for (int c = threadIdx.x + 256 * PER; c < each; c += 256) {
     const float g = y_row[c] * silu_m(z_row[c]);
     part = part + g * g;
   }
@@ -734,11 +764,11 @@ __global__ __launch_bounds__(256) void gated_parts_norm_kernel(const float* __re
   const float scale = 1.0f / sqrtf(total / (float)each + eps);
   T* dst = out + t * ldo + at;
 #pragma unroll
-  for (int j = 0; j < kGatedPer; ++j) {
+  for (int j = 0; j < PER; ++j) {
     const int c = threadIdx.x + 256 * j;
     if (c < each) dst[c] = from_f32<T>((mine[j] * scale) * weight[at + c]);
   }
-  for (int c = threadIdx.x + 256 * kGatedPer; c < each; c += 256)
+  for (int c = threadIdx.x + 256 * PER; c < each; c += 256)
     dst[c] = from_f32<T>(((y_row[c] * silu_m(z_row[c])) * scale) * weight[at + c]);
 }
 
@@ -900,14 +930,19 @@ extern "C" int ls_gated_parts_norm(int out_dtype, const float* y, long ldy, cons
   LS_REQUIRE(n_tokens > 0 && inner > 0 && parts > 0 && parts <= 65535 && inner % parts == 0 && ldy >= inner && ldz >= inner && ldo >= inner && eps > 0.f,
              "gated_parts_norm: %d elements in %d parts", inner, parts);
   LS_REQUIRE(y && z && weight && out, "gated_parts_norm: null operand");
+  LS_REQUIRE(out_dtype == kF32 || out_dtype == kBF16, "gated_parts_norm: unknown dtype %d", out_dtype);
   hipStream_t s = reinterpret_cast<hipStream_t>(stream);
-  if (out_dtype == kF32)
-    hipLaunchKernelGGL(gated_parts_norm_kernel<float>, dim3(n_tokens, parts), dim3(256), 0, s, y, ldy, z, ldz, inner / parts, weight,
-                       eps, (float*)out, ldo);
-  else if (out_dtype == kBF16)
-    hipLaunchKernelGGL(gated_parts_norm_kernel<bf16_t>, dim3(n_tokens, parts), dim3(256), 0, s, y, ldy, z, ldz, inner / parts, weight,
-                       eps, (bf16_t*)out, ldo);
-  else
-    return fail("gated_parts_norm: unknown dtype %d", out_dtype);
+  const int each = inner / parts;
+#define LS_GATED(T_, PER_)                                                                                                    \
+  hipLaunchKernelGGL((gated_parts_norm_kernel<T_, PER_>), dim3(n_tokens, parts), dim3(256), 0, s, y, ldy, z, ldz, each, weight, \
+                     eps, (T_*)out, ldo)
+#define LS_GATED_BY_SIZE(T_)             \
+  if (each <= 256) LS_GATED(T_, 1);      \
+  else if (each <= 1024) LS_GATED(T_, 4); \
+  else if (each <= 2048) LS_GATED(T_, 8); \
+  else LS_GATED(T_, 16);
+  if (out_dtype == kF32) { LS_GATED_BY_SIZE(float) } else { LS_GATED_BY_SIZE(bf16_t) }
+#undef LS_GATED_BY_SIZE
+#undef LS_GATED
   return check_launch("gated_parts_norm");
 }
