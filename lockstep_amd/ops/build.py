@@ -261,7 +261,7 @@ DEFAULT_TALKING_SHAPES = ((4, 2, 32, 16), (6, 3, 48, 24), (3, 1, 24, 40), (2, 2,
 #: (key size, value size) of the sink attention the tests and measurements use
 DEFAULT_SINK_SHAPES = ((16, 16), (32, 16), (24, 24), (40, 40), (32, 32), (24, 6), (128, 128),
                        (24, 40), (40, 32), (48, 36), (16, 6), (16, 8), (24, 8), (32, 48), (16, 24), (24, 16), (48, 32), (192, 128), (320, 256),
-                       (16, 40), (40, 24), (24, 20))
+                       (16, 40), (40, 24), (24, 20), (8, 4), (8, 8), (40, 6), (40, 8))
 
 
 def build_all(head_dims=DEFAULT_HEAD_DIMS, force: bool = True, mutants: bool = True,

@@ -136,3 +136,21 @@ def test_init_writes_a_tukavik_folder_from_its_preset(tmp_path):
         assert name in names, name
     assert "head" not in names and "l3.mix.dkv" not in names and "l2.mlp.up" not in names and "l1.mix.dq" not in names
     assert tuple(handle.shape("l3.dwa")) == (5,) and tuple(handle.shape("l1.mix.dkv")) == (40, 128)
+
+
+def test_init_writes_a_pozozen_folder_from_its_preset(tmp_path):
+    from lockstep_amd.config import PozozenConfig, config_from_dir
+    from lockstep_amd.weights import SafetensorsFile
+
+    done = run("init", "--preset", "pozozen-tiny", "--out", str(tmp_path / "k"), "--seed", "2")
+    assert done.returncode == 0, done.stderr
+    config = config_from_dir(tmp_path / "k")
+    assert isinstance(config, PozozenConfig) and config.width == 128 and config.order() == [0, 1, 2, 1, 2, 3]
+    handle = SafetensorsFile(tmp_path / "k" / "model.safetensors")
+    names = handle.keys()
+    for name in ("embed", "head", "final.norm", "final.norm.b", "l0.norm1.b", "l0.hc1.mix", "l0.mix.left.q.b", "l0.mix.right.in",
+                 "l0.mix.right.conv.b", "l0.mix.right.A_log", "l0.mlp.correction", "l0.mlp.e7.up", "l0.mlp.shared.down", "l1.mix.i.b",
+                 "l1.mix.norm", "l3.mix.g"):
+        assert name in names, name
+    assert "l0.mlp.e8.up" not in names and "l3.mlp.router" not in names and "l1.mix.left.q" not in names
+    assert tuple(handle.shape("l0.mlp.router")) == (10, 128) and tuple(handle.shape("l0.mix.right.conv")) == (256, 4)
