@@ -156,11 +156,18 @@ __global__ __launch_bounds__(256) void conv_ring_kernel(const float* __restrict_
 // tanh((logit + i_bias) / cap), f = logsigmoid(cap tanh((logit + f_bias) / cap)).  The running maximum m_t = max(f_t +
 // m_(t-1), i_t) starts at zero; la = f + m_(t-1) - m_t, b = exp(i - m_t), floor = exp(-m_t).  A wave a (request, head),
 // 64 tokens at a time: m_t as a function of the maximum in front is max(F + m, M), and such pairs are composed by moves
-// between lanes.  The state keeps m in two places a head, read at [q_start % 2] and left at [kv_len % 2] (a step of
-// single tokens then never writes what it reads).
+// between lanes.  m is kept and advanced in double: where a head forgets slowly, f is far below m's last place in float,
+// and what every token loses there would add up.  The state keeps m as the sum of two floats in two places a head, read at
+// [q_start % 2] and left at [kv_len % 2] (a step of single tokens then never writes what it reads).
 __device__ __forceinline__ void exp_gate_values(float zi, float zf, float cap, float& i, float& f) {
   i = cap * tanhf(zi / cap);
   f = log_sigmoid_m(cap * tanhf(zf / cap));
+}
+
+__device__ __forceinline__ double kept_maximum(const float* p) { return (double)p[0] + (double)p[1]; }
+__device__ __forceinline__ void keep_maximum(float* p, double m) {
+  p[0] = (float)m;
+  p[1] = (float)(m - (double)(float)m);
 }
 
 __global__ __launch_bounds__(64) void exp_gates_kernel(const float* __restrict__ raw, long ld, int i_at, int f_at, int H,
@@ -170,8 +177,8 @@ __global__ __launch_bounds__(64) void exp_gates_kernel(const float* __restrict__
   const int seq = blockIdx.x / H, h = blockIdx.x % H, lane = threadIdx.x;
   const SeqMeta m = seqs[seq];
   if (m.q_len <= 0) return;
-  float* kept = state + (long)m.table_row * state_stride + m_at + 2 * h;
-  float front = kept[m.q_start & 1];
+  float* kept = state + (long)m.table_row * state_stride + m_at + 4 * h;
+  double front = kept_maximum(kept + 2 * (m.q_start & 1));
   const float bi = i_bias[h], bf = f_bias[h];
   constexpr int AHEAD = 4;   // blocks of 64 tokens whose logits are on their way
   float zi[AHEAD], zf[AHEAD];
@@ -191,30 +198,30 @@ __global__ __launch_bounds__(64) void exp_gates_kernel(const float* __restrict__
       float i, f;
       exp_gate_values(zi[u] + bi, zf[u] + bf, cap, i, f);
       request(t0 + 64 * AHEAD, zi[u], zf[u]);
-      float F = in ? f : 0.f, M = in ? i : -3e38f;   // m behind this run of tokens: max(F + m in front, M)
+      double F = in ? (double)f : 0.0, M = in ? (double)i : -1e300;   // m behind this run of tokens: max(F + m in front, M)
 #pragma unroll
       for (int step = 1; step < 64; step <<= 1) {
-        const float oF = __shfl_up(F, step, kWave), oM = __shfl_up(M, step, kWave);
+        const double oF = __shfl_up(F, step, kWave), oM = __shfl_up(M, step, kWave);
         if (lane >= step) {
-          M = fmaxf(F + oM, M);
+          M = fmax(F + oM, M);
           F = F + oF;
         }
       }
-      const float mine = fmaxf(F + front, M);
-      float before = __shfl_up(mine, 1, kWave);
+      const double mine = fmax(F + front, M);
+      double before = __shfl_up(mine, 1, kWave);
       if (lane == 0) before = front;
       if (in) {
         Gate g;
-        g.la = fminf(f + before - mine, 0.f);
-        g.b = expf(i - mine);
-        g.floor = expf(-mine);
+        g.la = fminf((float)(((double)f + before) - mine), 0.f);
+        g.b = expf((float)((double)i - mine));
+        g.floor = expf((float)-mine);
         g.nq = 0.f;
         gates[(long)(m.q_off + t0 + lane) * H + h] = g;
       }
       front = __shfl(mine, 63, kWave);   // (lanes beyond the last token repeat its maximum: F and M are the identity there)
     }
   }
-  if (lane == 0) kept[m.kv_len & 1] = front;
+  if (lane == 0) keep_maximum(kept + 2 * (m.kv_len & 1), front);
 }
 
 // ---------------------------------------------------------------------------
@@ -427,13 +434,13 @@ __global__ __launch_bounds__(256) void memory_token_kernel(const float* __restri
     }
     float gi, gf;
     exp_gate_values(row[ex.i_at + h] + ex.i_bias[h], row[ex.f_at + h] + ex.f_bias[h], ex.cap, gi, gf);
-    float* kept = slot + ex.m_at + 2 * h;
-    const float before = kept[pos & 1];
-    const float now = fmaxf(gf + before, gi);
-    if (cb == 0 && threadIdx.x == 0) kept[(pos + 1) & 1] = now;
-    a = expf(fminf(gf + before - now, 0.f));
-    b = expf(gi - now);
-    floor = expf(-now);
+    float* kept = slot + ex.m_at + 4 * h;
+    const double before = kept_maximum(kept + 2 * (pos & 1));
+    const double now = fmax((double)gf + before, (double)gi);
+    if (cb == 0 && threadIdx.x == 0) keep_maximum(kept + 2 * ((pos + 1) & 1), now);
+    a = expf(fminf((float)(((double)gf + before) - now), 0.f));
+    b = expf((float)((double)gi - now));
+    floor = expf((float)-now);
   }
   __syncthreads();
   float kk[R], qq[R];
@@ -807,7 +814,7 @@ extern "C" int ls_exp_gates(const float* raw, long ld, int i_at, int f_at, int H
                             const void* seqs, int n_seqs, float* state, long state_stride, long m_at, float* gates, void* stream) {
   LS_REQUIRE(n_seqs > 0 && H > 0 && cap > 0.f && i_at >= 0 && f_at >= 0 && ld >= (long)i_at + H && ld >= (long)f_at + H,
              "exp_gates: bad sizes");
-  LS_REQUIRE(m_at >= 0 && state_stride >= m_at + 2L * H, "exp_gates: the state holds no running maxima");
+  LS_REQUIRE(m_at >= 0 && state_stride >= m_at + 4L * H, "exp_gates: the state holds no running maxima");
   LS_REQUIRE(raw && i_bias && f_bias && seqs && state && gates && aligned16(gates), "exp_gates: bad operands");
   hipLaunchKernelGGL(exp_gates_kernel, dim3(n_seqs * H), dim3(64), 0, reinterpret_cast<hipStream_t>(stream), raw, ld, i_at, f_at, H,
                      i_bias, f_bias, cap, (const SeqMeta*)seqs, state, state_stride, m_at, (Gate*)gates);
@@ -878,7 +885,7 @@ extern "C" int ls_exp_token(const float* raw, long ld, int q_at, int k_at, int v
   LS_REQUIRE(q_at >= 0 && k_at >= 0 && v_at >= 0 && i_at >= 0 && f_at >= 0 && ld >= (long)q_at + (long)H * N && ld >= (long)k_at + (long)H * N &&
                  ld >= (long)v_at + (long)H * DV && ld >= (long)i_at + H && ld >= (long)f_at + H,
              "exp_token: the projections do not fit the rows");
-  LS_REQUIRE(m_at >= (long)H * N * DV + (long)H * N && state_stride >= m_at + 2L * H && ldo >= (long)H * DV, "exp_token: state or output too short");
+  LS_REQUIRE(m_at >= (long)H * N * DV + (long)H * N && state_stride >= m_at + 4L * H && ldo >= (long)H * DV, "exp_token: state or output too short");
   LS_REQUIRE(raw && i_bias && f_bias && seqs && state && gates && out, "exp_token: null operand");
   hipStream_t s = reinterpret_cast<hipStream_t>(stream);
   const SpaceArgs sp{};

@@ -151,7 +151,7 @@ int ls_conv_gates(const float* raw, long ld, int x_at, int dt_at, int n_tokens, 
                   const float* bias, const float* a_log, const float* dt_bias, const int* tok_seq, const int* tok_pos,
                   const void* seqs, int n_seqs, float* state, long state_stride, long ring_at, float* conv, float* gates,
                   void* stream);
-// Exponential gates with a running maximum, kept as two numbers a head at m_at in the state.
+// Exponential gates with a running maximum, kept as two sums of two floats a head at m_at in the state.
 int ls_exp_gates(const float* raw, long ld, int i_at, int f_at, int H, const float* i_bias, const float* f_bias, float cap,
                  const void* seqs, int n_seqs, float* state, long state_stride, long m_at, float* gates, void* stream);
 // Token by token, for the requests of at most `longest` tokens.

@@ -1688,12 +1688,12 @@ class Kernels:
                   state: torch.Tensor, max_at: int, gates: torch.Tensor) -> None:
         """Exponential gates: ``i = cap tanh((raw[i_at ..] + i_bias) / cap)``, ``f = logsigmoid(cap tanh((raw[f_at ..] + f_bias) /
         cap))``, a running maximum ``m = max(f + m, i)`` from zero; ``log a = f + m_before - m``, ``b = exp(i - m)``, floor
-        ``exp(-m)``.  ``state``: at ``max_at`` two numbers a head, of which the one of the length's parity is the maximum."""
+        ``exp(-m)``.  ``state``: at ``max_at`` two places of two floats a head, the maximum being the sum in the one of the length's parity."""
         _rows_ok(raw, "exp_gates raw")
         if not (raw.dtype == torch.float32 and cap > 0 and min(i_at, f_at) >= 0 and raw.shape[1] >= max(i_at, f_at) + heads):
             raise KernelError("exp_gates: the projections do not fit the float32 rows, or the cap is not positive")
         self._f32_vector(i_bias, heads, "exp_gates i_bias"); self._f32_vector(f_bias, heads, "exp_gates f_bias")
-        self._memory_state(state, max_at + 2 * heads, "exp_gates")
+        self._memory_state(state, max_at + 4 * heads, "exp_gates")
         self._gates_ok(gates, raw.shape[0], heads, "exp_gates")
         self._seqs_ok(seqs, n_seqs, "exp_gates")
         if raw.shape[0] == 0:
@@ -1785,7 +1785,7 @@ class Kernels:
                 and raw.shape[1] >= max(max(q_at, k_at) + heads * rows, v_at + heads * vdim, max(i_at, f_at) + heads)):
             raise KernelError("exp_token: the projections do not fit the float32 rows, or the cap is not positive")
         self._f32_vector(i_bias, heads, "exp_token i_bias"); self._f32_vector(f_bias, heads, "exp_token f_bias")
-        self._memory_state(state, max_at + 2 * heads, "exp_token")
+        self._memory_state(state, max_at + 4 * heads, "exp_token")
         self._gates_ok(gates, n_seqs, heads, "exp_token")
         self._seqs_ok(seqs, n_seqs, "exp_token")
         if not (out.dtype == torch.float32 and tuple(out.shape) == (n_seqs, heads * vdim)):

@@ -198,7 +198,8 @@ class MatrixMemory(_Memory):
 
     Parameters: ``hidden_size``, ``num_heads``, ``head_dim``, ``value_dim``, ``gate_cap``, ``eps``, ``denom_eps``, ``out_scale``.  Tensors below
     the prefix: ``q``, ``k``, ``v``, ``g``, ``i``, ``i.b``, ``f``, ``f.b``, ``norm``, ``o``.  A request's state slot holds ``S``, ``n`` and, in two places a
-    head of which the length's parity says the current one, the maximum."""
+    head of which the length's parity says the current one, the maximum, as the sum of two numbers (a slow forget gate is far
+    below the maximum's last place in float32)."""
 
     norm = True
 
@@ -221,7 +222,7 @@ class MatrixMemory(_Memory):
                 WeightSpec(f"{prefix}.norm", (n * dv,), kind="vector", init="norm"), WeightSpec(f"{prefix}.o", (h, n * dv))]
 
     def cache_spec(self):
-        return StateSpec((-(-(self.max_at + 2 * self.heads) // 4) * 4,), "float32")
+        return StateSpec((-(-(self.max_at + 4 * self.heads) // 4) * 4,), "float32")
 
     def in_matrices(self, weights) -> list:
         return [weights.get(f"{self.prefix}.{n}") for n in "qkvgif"]

@@ -120,7 +120,7 @@ def test_cache_units_of_every_pass_and_of_both_halves_of_a_parallel_mixer():
     from lockstep_amd.parts import PagedKVSpec, StateSpec
 
     units = cache_units(CASES["A"]["raw"])
-    assert units[0] == StateSpec((-(-(3 * 20 * 25 + 6) // 4) * 4,), "float32")      # S, n and the maxima
+    assert units[0] == StateSpec((3 * 20 * 25 + 12,), "float32")      # S, n and the maxima
     assert units[1] == units[4] == PagedKVSpec(2, 24, 21, value_dim=16)
     assert units[2] == units[5] == StateSpec((4 * 24 * 16 + 3 * 160,), "float32")    # S and the ring of the convolution's inputs
     assert units[7] == PagedKVSpec(3, 16, None, value_dim=24)

@@ -31,8 +31,8 @@ F64 = torch.float64
 # Bounds on max |engine - plain| / max |plain logit| over a request, some three times the largest error
 # measured on the MI355X on these weights.  A matrix memory's read-out whose terms nearly cancel is a short vector, which the norm
 # behind it lengthens together with its rounding: in float32 one position in a hundred may go up to FAR times beyond.
-TOL = {"float32": 1.5e-5, "bfloat16": 4e-2}
-FAR = 6
+TOL = {"float32": 6e-6, "bfloat16": 4e-2}
+FAR = 7
 
 
 def K():
@@ -289,8 +289,8 @@ def test_the_matrix_memory_over_unequal_requests_in_steps(dtype, heads, rows, dv
         err = (got[s].double() - want).abs().max(dim=1)[0] / want.abs().max()
         print(heads, rows, dv, dtype, s, f"{float(err.max()):.2e}")
         # (gates that are open as far as the cap lets them make sums whose terms nearly cancel; see FAR)
-        assert float(err.median()) < (2e-6 if dtype == torch.float32 else 2e-3)
-        assert float(err.max()) < (1e-4 if dtype == torch.float32 else 1e-2), (s, int(err.argmax()))
+        assert float(err.median()) < (1e-6 if dtype == torch.float32 else 2e-3)
+        assert float(err.max()) < (4e-5 if dtype == torch.float32 else 1e-2), (s, int(err.argmax()))
 
 
 @pytest.mark.parametrize("tokens, routed, top, groups, keep", [(1, 8, 2, 4, 2), (9, 18, 3, 3, 1), (40, 12, 12, 1, 1), (700, 15, 4, 5, 2), (33, 100, 6, 10, 3),
