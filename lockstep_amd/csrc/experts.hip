@@ -25,6 +25,8 @@
 
 #include "common.h"
 
+#include <type_traits>
+
 namespace ls {
 
 constexpr int kMaxTop = 16;
@@ -63,15 +65,23 @@ __device__ __forceinline__ void keep_better_of(float& v, int& e) {
               __builtin_amdgcn_mov_dpp(e, CTRL, 0xF, 0xF, true));
 }
 
-// PL: experts a lane holds
+// A lane's entries of a vector over the experts (null: zeros).
 template <int PL>
-__device__ __forceinline__ void pick_top(const float* __restrict__ row, const float* __restrict__ bias, int E, int top,
-                                         int lane, int* __restrict__ picked, float* __restrict__ share, const Choice& how) {
+__device__ __forceinline__ void lane_entries(const float* __restrict__ of, int E, int lane, float (&mine)[PL]) {
+#pragma unroll
+  for (int m = 0; m < PL; ++m) mine[m] = of && lane + 64 * m < E ? of[lane + 64 * m] : 0.f;
+}
+
+// PL: experts a lane holds; bias and correction: their entries
+template <int PL>
+__device__ __forceinline__ void pick_top(const float* __restrict__ row, const float (&bias)[PL], const float (&correction)[PL],
+                                         int E, int top, int lane, int* __restrict__ picked, float* __restrict__ share,
+                                         const Choice& how) {
   float mine[PL], score[PL];
 #pragma unroll
   for (int m = 0; m < PL; ++m) {
     const int e = lane + 64 * m;
-    mine[m] = e < E ? row[e] + (bias ? bias[e] : 0.f) : 0.f;
+    mine[m] = e < E ? row[e] + bias[m] : 0.f;
     score[m] = 0.f;
   }
   // the largest of every lane's open experts, the lower index winning a tie (0x7fffffff: none is open)
@@ -110,7 +120,7 @@ __device__ __forceinline__ void pick_top(const float* __restrict__ row, const fl
 #pragma unroll
     for (int m = 0; m < PL; ++m) {
       score[m] = score[m] * inv;
-      if (lane + 64 * m < E) mine[m] = score[m] + how.correction[lane + 64 * m];
+      if (lane + 64 * m < E) mine[m] = score[m] + correction[m];
     }
     if (how.keep < how.groups) {   // the groups, best first: every pick closes its group for the next one
       const int each = E / how.groups;
@@ -178,7 +188,11 @@ __global__ __launch_bounds__(256) void route_topk_kernel(const float* __restrict
                                                          int* __restrict__ expert, float* __restrict__ weight, Choice how) {
   const int t = blockIdx.x * 4 + (threadIdx.x >> 6);
   if (t >= n_tokens) return;
-  pick_top<PL>(z + (long)t * ldz, bias, E, top, threadIdx.x & 63, expert + (long)t * top, weight + (long)t * top, how);
+  const int lane = threadIdx.x & 63;
+  float own_bias[PL], own_correction[PL];
+  lane_entries<PL>(bias, E, lane, own_bias);
+  lane_entries<PL>(how.correction, E, lane, own_correction);
+  pick_top<PL>(z + (long)t * ldz, own_bias, own_correction, E, top, lane, expert + (long)t * top, weight + (long)t * top, how);
 }
 
 // ---------------------------------------------------------------------------
@@ -255,42 +269,87 @@ __global__ __launch_bounds__(64) void route_place_kernel(const int* __restrict__
   place_pairs(expert, counts, P, E, blockIdx.x, threadIdx.x, rows_a_tile, order, tiles, cap);
 }
 
+// A barrier between LDS writes and reads that waits for this wave's LDS operations only: loads from memory (and stores
+// to it) stay on their way across it.
+__device__ __forceinline__ void lds_barrier() { __asm__ volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
+
 constexpr int kSmallPairs = 512, kSmallExperts = 512;   // what the one-workgroup kernel keeps in LDS
 
-template <int PL>
+constexpr int kProductTiles = 8;    // tiles of 16 experts whose logits the one-workgroup kernel forms itself
+
+// PRODUCT: the logits come from up to 16 rows of x and the router's matrix [E][K] instead of z
+template <int PL, typename T, bool PRODUCT>
 __global__ __launch_bounds__(1024) void route_small_kernel(const float* __restrict__ z, long ldz,
                                                            const float* __restrict__ bias, int n_tokens, int E, int top,
                                                            int rows_a_tile, int* __restrict__ expert,
                                                            float* __restrict__ weight, int* __restrict__ order,
                                                            int* __restrict__ tiles, int cap,
                                                            const int* __restrict__ token_ids, const int* __restrict__ table,
-                                                           Choice how) {
+                                                           Choice how, const T* __restrict__ x, long ldx,
+                                                           const T* __restrict__ w_router, int K) {
   __shared__ int picks_s[kSmallPairs];
-  __shared__ float share_s[16][kMaxTop];
+  __shared__ float share_s[kSmallPairs];
   __shared__ int counts_s[kSmallExperts];
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
   const int P = n_tokens * top;
+  float own_bias[PL], own_correction[PL];
+  lane_entries<PL>(bias, E, lane, own_bias);
+  lane_entries<PL>(how.correction, E, lane, own_correction);
+  if constexpr (PRODUCT) {   // the logits first: z = x W^T, the column tiles and cuts of K dealt to the sixteen waves
+    __shared__ f32x4 sums_s[16][64];
+    __shared__ float z_s[16][16 * kProductTiles];
+    constexpr int VEC = Atom<T>::VEC, KC = Atom<T>::KCHUNK, U = 8;
+    const int l16 = lane & 15, quad = lane >> 4;
+    const int tiles16 = (E + 15) / 16, cuts = 16 / tiles16;
+    const int ct = w % tiles16, cut = w / tiles16;
+    f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+    if (cut < cuts) {
+      const bool w_ok = 16 * ct + l16 < E, x_ok = l16 < n_tokens;
+      const T* w_row = w_router + (long)(w_ok ? 16 * ct + l16 : 0) * K;
+      const T* x_row = x + (long)(x_ok ? l16 : 0) * ldx;
+      const int each = (K + KC * cuts - 1) / (KC * cuts) * KC;
+      const int hi = min(K, (cut + 1) * each);
+      for (int k0 = cut * each; k0 < hi; k0 += U * KC) {
+        typename Atom<T>::vec_t a[U], b[U];
+#pragma unroll
+        for (int u = 0; u < U; ++u) {
+          a[u] = load_vec<T>(w_row, 0, k0 + u * KC + VEC * quad, hi, 0, w_ok, true);
+          b[u] = load_vec<T>(x_row, 0, k0 + u * KC + VEC * quad, hi, 0, x_ok, true);
+        }
+#pragma unroll
+        for (int u = 0; u < U; ++u) Atom<T>::mma(acc, a[u], b[u]);
+      }
+    }
+    sums_s[w][lane] = acc;
+    lds_barrier();
+    if (w < tiles16) {   // (the cuts in ascending order)
+      f32x4 sum = sums_s[w][lane];
+      for (int o = 1; o < cuts; ++o) sum = sum + sums_s[w + o * tiles16][lane];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) z_s[l16][16 * w + 4 * quad + i] = sum[i];
+    }
+    lds_barrier();
+    z = &z_s[0][0];
+    ldz = 16 * kProductTiles;
+  }
   if (table) {   // the picks are looked up, not chosen
     for (int pair = threadIdx.x; pair < P; pair += 1024) {
-      const int e = table[(long)token_ids[pair / top] * top + pair % top];
-      picks_s[pair] = e;
-      expert[pair] = e;
-      weight[pair] = 1.0f / (float)top;
+      picks_s[pair] = table[(long)token_ids[pair / top] * top + pair % top];
+      share_s[pair] = 1.0f / (float)top;
     }
   }
-  for (int t = w; t < n_tokens && !table; t += 16) {
-    pick_top<PL>(z + (long)t * ldz, bias, E, top, lane, picks_s + t * top, share_s[w], how);
-    if (lane < top) {
-      expert[(long)t * top + lane] = picks_s[t * top + lane];
-      weight[(long)t * top + lane] = share_s[w][lane];
-    }
+  for (int t = w; t < n_tokens && !table; t += 16)
+    pick_top<PL>(z + (long)t * ldz, own_bias, own_correction, E, top, lane, picks_s + t * top, share_s + t * top, how);
+  lds_barrier();
+  for (int pair = threadIdx.x; pair < P; pair += 1024) {
+    expert[pair] = picks_s[pair];
+    weight[pair] = share_s[pair];
   }
-  __syncthreads();
   for (int e = w; e < E; e += 16) {
     const int n = count_pairs(picks_s, P, e, lane);
     if (lane == 0) counts_s[e] = n;
   }
-  __syncthreads();
+  lds_barrier();
   for (int e = w; e < E; e += 16) place_pairs(picks_s, counts_s, P, E, e, lane, rows_a_tile, order, tiles, cap);
 }
 
@@ -298,35 +357,51 @@ __global__ __launch_bounds__(1024) void route_small_kernel(const float* __restri
 // (3) act [P][ldy] (T) = act(x[token] W_gate[e]^T, x[token] W_up[e]^T) for the pairs of every tile, in the
 // order of `order`.  w_gate, w_up [E][F][K].  A workgroup: one tile, four waves with 16 columns of F each.
 // ---------------------------------------------------------------------------
+// An expert that every token uses, worked on beside the routed ones in the launches of small steps: work items from `at`
+// on are tiles of 16 tokens.  w_gate_up holds its rows interleaved in tiles of 16 (gate, up, gate, ...; the last tile padded
+// with zeros), w_down [N][F]; the plain gated unit silu(g) u; act [n_tokens][ldy] scratch, out [n_tokens][N] float.
+template <typename T>
+struct SharedExpert {
+  const T* w_gate_up;
+  const T* w_down;
+  int F, at;   // at: the routed experts' work items (0x7fffffff: there is no such expert)
+  T* act;
+  long ldy;
+  float* out;
+};
+
 template <typename T, int RT, int KS>
 __global__ __launch_bounds__(256) void experts_gate_up_kernel(const T* __restrict__ x, long ldx,
                                                               const T* __restrict__ w_gate, const T* __restrict__ w_up,
                                                               int F, int K, int top, const int* __restrict__ order,
                                                               const int* __restrict__ tiles, float limit, float alpha, float shift,
                                                               const float* __restrict__ in_weight, T* __restrict__ act, long ldy,
-                                                              int real) {
+                                                              int real, int n_tokens, SharedExpert<T> sh) {
   // in_weight (or null): a pair's routing weight multiplies the expert's input, w * x, so both products are scaled
   // by it before the gated unit (the down product then adds the expert's output as it is)
   constexpr int VEC = Atom<T>::VEC, KC = Atom<T>::KCHUNK;
-  const int e = tiles[4 * blockIdx.x];
+  const bool all = KS > 1 && (int)blockIdx.x >= sh.at;   // (the same for the whole workgroup)
+  const int e = all ? 0 : tiles[4 * blockIdx.x];
   if (e < 0 || e >= real) return;   // (an expert that returns its input has nothing to multiply)
-  const int first = tiles[4 * blockIdx.x + 1], rows = tiles[4 * blockIdx.x + 2];
+  const int first = all ? 16 * ((int)blockIdx.x - sh.at) : tiles[4 * blockIdx.x + 1];
+  const int rows = all ? min(16, n_tokens - first) : tiles[4 * blockIdx.x + 2];
+  if (all) F = sh.F;
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
   const int l16 = lane & 15, quad = lane >> 4;
   // KS 1: the four waves take 16 columns each.  KS 4 (few rows): they take a quarter of K each for the same 16
   // columns, so that all of a wave's operands are on their way at once, and their sums are added in wave order.
   const int col0 = KS == 1 ? (blockIdx.y * 4 + w) * 16 : blockIdx.y * 16;
   if (col0 >= F) return;
-  const bool w_ok = col0 + l16 < F;
-  const T* g_row = w_gate + ((long)e * F + (w_ok ? col0 + l16 : 0)) * K;
-  const T* u_row = w_up + ((long)e * F + (w_ok ? col0 + l16 : 0)) * K;
+  const bool w_ok = all || col0 + l16 < F;
+  const T* g_row = all ? sh.w_gate_up + (long)(2 * col0 + l16) * K : w_gate + ((long)e * F + (w_ok ? col0 + l16 : 0)) * K;
+  const T* u_row = all ? g_row + 16L * K : w_up + ((long)e * F + (w_ok ? col0 + l16 : 0)) * K;
   const T* x_row[RT];
   bool x_ok[RT];
 #pragma unroll
   for (int r = 0; r < RT; ++r) {
     x_ok[r] = 16 * r + l16 < rows;
-    const int pair = x_ok[r] ? order[first + 16 * r + l16] : 0;
-    x_row[r] = x + (long)(pair / top) * ldx;
+    const int token = all ? first + l16 : (x_ok[r] ? order[first + 16 * r + l16] : 0) / top;
+    x_row[r] = x + (long)(x_ok[r] ? token : 0) * ldx;
   }
   f32x4 acc_g[RT], acc_u[RT];
 #pragma unroll
@@ -376,12 +451,16 @@ __global__ __launch_bounds__(256) void experts_gate_up_kernel(const T* __restric
 #pragma unroll
   for (int r = 0; r < RT; ++r) {
     if (!x_ok[r]) continue;
-    T* dst = act + (long)(first + 16 * r + l16) * ldy;
-    const float wt = in_weight ? in_weight[order[first + 16 * r + l16]] : 1.0f;
+    T* dst = all ? sh.act + (long)(first + l16) * sh.ldy : act + (long)(first + 16 * r + l16) * ldy;
+    const float wt = in_weight && !all ? in_weight[order[first + 16 * r + l16]] : 1.0f;
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       const int c = col0 + 4 * quad + i;
       if (c < F) {
+        if (all) {
+          dst[c] = from_f32<T>((acc_g[r][i] * sigmoid_e(acc_g[r][i])) * acc_u[r][i]);
+          continue;
+        }
         const float g = fminf(acc_g[r][i] * wt, limit);
         const float u = fminf(fmaxf(acc_u[r][i] * wt, -limit), limit);
         dst[c] = from_f32<T>((g * sigmoid_e(alpha * g)) * (u + shift));
@@ -413,11 +492,19 @@ __global__ __launch_bounds__(256) void experts_down_kernel(const T* __restrict__
                                                            const int* __restrict__ tiles,
                                                            const float* __restrict__ weight, float* __restrict__ P,
                                                            const T* __restrict__ x, long ldx, const float* __restrict__ share,
-                                                           int real) {
+                                                           int real, SharedExpert<T> sh) {
   constexpr int VEC = Atom<T>::VEC, KC = Atom<T>::KCHUNK;
-  const int e = tiles[4 * blockIdx.x];
+  const bool all = KS > 1 && (int)blockIdx.x >= sh.at;
+  const int e = all ? 0 : tiles[4 * blockIdx.x];
   if (e < 0) return;
-  const int first = tiles[4 * blockIdx.x + 1], rows = tiles[4 * blockIdx.x + 2];
+  const int first = all ? 16 * ((int)blockIdx.x - sh.at) : tiles[4 * blockIdx.x + 1];
+  const int rows = all ? min(16, n_tokens - first) : tiles[4 * blockIdx.x + 2];
+  if (all) {
+    F = sh.F;
+    ldy = sh.ldy;
+    act = sh.act;
+    w_down = sh.w_down;
+  }
   if (e >= real) {   // (the whole workgroup)
     constexpr int kCols = KS == 1 ? 64 : 16;
     pass_input<T>(x, ldx, share, first, rows, blockIdx.y * kCols, min(N, (int)(blockIdx.y + 1) * kCols), top, n_tokens, N, order, P);
@@ -473,13 +560,13 @@ __global__ __launch_bounds__(256) void experts_down_kernel(const T* __restrict__
 #pragma unroll
   for (int r = 0; r < RT; ++r) {
     if (!y_ok[r]) continue;
-    const int pair = order[first + 16 * r + l16];
-    const float share = weight ? weight[pair] : 1.0f;
-    float* dst = P + ((long)(pair % top) * n_tokens + pair / top) * N;
+    const int pair = all ? 0 : order[first + 16 * r + l16];
+    const float factor = weight && !all ? weight[pair] : 1.0f;
+    float* dst = all ? sh.out + (long)(first + l16) * N : P + ((long)(pair % top) * n_tokens + pair / top) * N;
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       const int c = col0 + 4 * quad + i;
-      if (c < N) dst[c] = share * acc[r][i];
+      if (c < N) dst[c] = factor * acc[r][i];
     }
   }
 }
@@ -691,8 +778,9 @@ extern "C" int ls_experts_route(const float* z, long ldz, const float* bias, int
   const int P = n_tokens * top;
 #define LS_ROUTE(PL_)                                                                                                     \
   if (P <= kSmallPairs && E <= kSmallExperts)                                                                             \
-    hipLaunchKernelGGL(route_small_kernel<PL_>, dim3(1), dim3(1024), 0, s, z, ldz, bias, n_tokens, E, top, rows_a_tile,   \
-                       expert, weight, order, tiles, cap, (const int*)nullptr, (const int*)nullptr, how);                 \
+    hipLaunchKernelGGL((route_small_kernel<PL_, float, false>), dim3(1), dim3(1024), 0, s, z, ldz, bias, n_tokens, E, top, \
+                       rows_a_tile, expert, weight, order, tiles, cap, (const int*)nullptr, (const int*)nullptr, how,     \
+                       (const float*)nullptr, 0L, (const float*)nullptr, 0);                                              \
   else                                                                                                                    \
     hipLaunchKernelGGL(route_topk_kernel<PL_>, dim3((n_tokens + 3) / 4), dim3(256), 0, s, z, ldz, bias, n_tokens, E, top, \
                        expert, weight, how);
@@ -707,6 +795,43 @@ extern "C" int ls_experts_route(const float* z, long ldz, const float* bias, int
   return check_launch("experts_route");
 }
 
+// Whether ls_experts_route_product takes a step of n_tokens tokens.
+extern "C" int ls_experts_route_product_ok(int dtype, int n_tokens, int E, int top, int K) {
+  return n_tokens <= 16 && E <= 16 * kProductTiles && (long)n_tokens * top <= kSmallPairs && K % (dtype == kF32 ? 4 : 8) == 0;
+}
+
+// The same with the router's product inside: x [n_tokens][ldx] and w_router [E][K] of the compute dtype instead of logits.
+extern "C" int ls_experts_route_product(int dtype, const void* x, long ldx, const void* w_router, int K, const float* bias,
+                                        int n_tokens, int E, int top, int rows_a_tile, int* expert, float* weight, int* order,
+                                        int* tiles, int cap, int scoring, const float* correction, int groups, int keep,
+                                        void* stream) {
+  LS_REQUIRE(scoring >= 0 && scoring <= 2, "experts_route_product: scoring %d", scoring);
+  LS_REQUIRE(scoring != 2 || (correction && groups > 0 && keep > 0 && keep <= groups && E % groups == 0 && top <= keep * (E / groups)),
+             "experts_route_product: %d experts in %d groups of which %d are kept, %d a token", E, groups, keep, top);
+  LS_REQUIRE(n_tokens > 0 && E > 0 && top > 0 && top <= E && top <= kMaxTop && K > 0 && ldx >= K && ls_experts_route_product_ok(dtype, n_tokens, E, top, K),
+             "experts_route_product: %d tokens, %d experts, %d chosen", n_tokens, E, top);
+  LS_REQUIRE(rows_a_tile == 16 || rows_a_tile == 32 || rows_a_tile == 64, "experts_route_product: tiles of %d rows", rows_a_tile);
+  LS_REQUIRE(x && w_router && expert && weight && order && tiles && cap >= ls_experts_tile_capacity(n_tokens, E, top, rows_a_tile),
+             "experts_route_product: bad operands");
+  LS_REQUIRE(dtype == kF32 || dtype == kBF16, "experts_route_product: unknown dtype %d", dtype);
+  LS_REQUIRE(reinterpret_cast<uintptr_t>(x) % 16 == 0 && reinterpret_cast<uintptr_t>(w_router) % 16 == 0 &&
+                 ldx % (dtype == kF32 ? 4 : 8) == 0,
+             "experts_route_product: operands must be 16-byte aligned");
+  hipStream_t s = reinterpret_cast<hipStream_t>(stream);
+  const Choice how{scoring, groups, keep, correction};
+#define LS_ROUTE_PRODUCT(PL_, T_)                                                                                         \
+  hipLaunchKernelGGL((route_small_kernel<PL_, T_, true>), dim3(1), dim3(1024), 0, s, (const float*)nullptr, 0L, bias, n_tokens, E, \
+                     top, rows_a_tile, expert, weight, order, tiles, cap, (const int*)nullptr, (const int*)nullptr, how,  \
+                     (const T_*)x, ldx, (const T_*)w_router, K)
+  if (dtype == kF32) {
+    if (E <= 64) LS_ROUTE_PRODUCT(1, float); else LS_ROUTE_PRODUCT(2, float);
+  } else {
+    if (E <= 64) LS_ROUTE_PRODUCT(1, bf16_t); else LS_ROUTE_PRODUCT(2, bf16_t);
+  }
+#undef LS_ROUTE_PRODUCT
+  return check_launch("experts_route_product");
+}
+
 // The same grouping for experts that a table names: token_ids [n_tokens], table [vocab][top] with entries in [0, E).
 extern "C" int ls_experts_route_table(const int* token_ids, const int* table, int n_tokens, int E, int top,
                                       int rows_a_tile, int* expert, float* weight, int* order, int* tiles, int cap,
@@ -718,8 +843,9 @@ extern "C" int ls_experts_route_table(const int* token_ids, const int* table, in
   hipStream_t s = reinterpret_cast<hipStream_t>(stream);
   const int P = n_tokens * top;
   if (P <= kSmallPairs && E <= kSmallExperts) {
-    hipLaunchKernelGGL(route_small_kernel<1>, dim3(1), dim3(1024), 0, s, (const float*)nullptr, 0L, (const float*)nullptr,
-                       n_tokens, E, top, rows_a_tile, expert, weight, order, tiles, cap, token_ids, table, Choice{0, 1, 1, nullptr});
+    hipLaunchKernelGGL((route_small_kernel<1, float, false>), dim3(1), dim3(1024), 0, s, (const float*)nullptr, 0L, (const float*)nullptr,
+                       n_tokens, E, top, rows_a_tile, expert, weight, order, tiles, cap, token_ids, table, Choice{0, 1, 1, nullptr},
+                       (const float*)nullptr, 0L, (const float*)nullptr, 0);
   } else {
     hipLaunchKernelGGL(route_table_kernel, dim3((P + 255) / 256), dim3(256), 0, s, token_ids, table, n_tokens, top, expert,
                        weight);
@@ -735,7 +861,14 @@ extern "C" int ls_experts_apply(int dtype, const void* x, long ldx, const void* 
                                 const void* w_down, int n_tokens, int E, int top, int K, int F, int N,
                                 int rows_a_tile, const int* order, const int* tiles, int cap, const float* weight,
                                 float limit, float alpha, float shift, void* act, long ldy, float* P, int weigh_input,
-                                int real, void* stream) {
+                                int real, const void* sh_gate_up, const void* sh_down, int sh_F, void* sh_act, long sh_ldy,
+                                float* sh_out, void* stream) {
+  // sh_*: an expert that every token uses, worked on in the same launches (tiles of 16 rows only; null: none)
+  const bool with_shared = sh_gate_up != nullptr;
+  LS_REQUIRE(!with_shared || (rows_a_tile == 16 && sh_down && sh_act && sh_out && sh_F > 0 && sh_ldy >= sh_F &&
+                              reinterpret_cast<uintptr_t>(sh_gate_up) % 16 == 0 && reinterpret_cast<uintptr_t>(sh_down) % 16 == 0 &&
+                              reinterpret_cast<uintptr_t>(sh_act) % 16 == 0),
+             "experts_apply: a shared expert is worked on beside tiles of 16 rows, its operands 16-byte aligned");
   // weigh_input: the routing weight multiplies the expert's input instead of its output.  real: experts from this one on
   // (of the E that the tiles may name) have no weights and return their input
   LS_REQUIRE(real > 0 && real <= E && (real == E || K == N), "experts_apply: %d of %d experts with weights", real, E);
@@ -754,14 +887,20 @@ extern "C" int ls_experts_apply(int dtype, const void* x, long ldx, const void* 
   hipStream_t s = reinterpret_cast<hipStream_t>(stream);
   // tiles of 16 rows (few tokens an expert): a workgroup takes 16 columns and cuts K over its waves
   const int cols = rows_a_tile == 16 ? 16 : 64;
-  const dim3 grid_up(cap, (F + cols - 1) / cols), grid_down(cap, (N + cols - 1) / cols);
+  const int more = with_shared ? (n_tokens + 15) / 16 : 0, widest = with_shared && sh_F > F ? sh_F : F;
+  const dim3 grid_up(cap + more, (widest + cols - 1) / cols), grid_down(cap + more, (N + cols - 1) / cols);
+  auto shared_of = [&](auto* of_type) {
+    typedef std::remove_pointer_t<decltype(of_type)> E_;
+    return SharedExpert<E_>{(const E_*)sh_gate_up, (const E_*)sh_down, sh_F, with_shared ? cap : 0x7fffffff, (E_*)sh_act, sh_ldy, sh_out};
+  };
 #define LS_EXPERTS(T_, RT_, KS_)                                                                                      \
   do {                                                                                                                \
     hipLaunchKernelGGL((experts_gate_up_kernel<T_, RT_, KS_>), grid_up, dim3(256), 0, s, (const T_*)x, ldx,           \
                        (const T_*)w_gate, (const T_*)w_up, F, K, top, order, tiles, limit, alpha, shift, in_weight,   \
-                       (T_*)act, ldy, real);                                                                          \
+                       (T_*)act, ldy, real, n_tokens, shared_of((T_*)nullptr));                                       \
     hipLaunchKernelGGL((experts_down_kernel<T_, RT_, KS_>), grid_down, dim3(256), 0, s, (const T_*)act, ldy,          \
-                       (const T_*)w_down, N, F, top, n_tokens, order, tiles, out_weight, P, (const T_*)x, ldx, weight, real); \
+                       (const T_*)w_down, N, F, top, n_tokens, order, tiles, out_weight, P, (const T_*)x, ldx, weight, real, \
+                       shared_of((T_*)nullptr));                                                                      \
   } while (0)
   // tiles of 64 rows go through LDS where every row of every operand starts on a 16-byte boundary
   const bool staged = rows_a_tile == 64 && K % vec == 0 && F % vec == 0 && ldx % vec == 0 && ldy % vec == 0;

@@ -351,6 +351,8 @@ __global__ __launch_bounds__(256) void memory_walk_kernel(HeadRows q, HeadRows k
 //   C itself (M inputs a channel), and one workgroup of those that read a channel leaves the token's input in the ring,
 //   in a row that no one reads in this step.
 // else: q, k, v as they are in raw (q_at, k_at, v_at), exponential gates as exp_gates_kernel forms them.
+// WHOLE: a workgroup takes all columns of a head (256 threads for every 32 of them, at most 128 columns), divides the head by
+// its denominator and its root mean square and multiplies it by the weight and the gate's sigmoid; normed [T][ldn] (T).
 // ---------------------------------------------------------------------------
 struct SpaceArgs {
   int x_at, dt_at, C, G, M;
@@ -362,37 +364,57 @@ struct ExpArgs {
   long m_at;
   float cap, q_scale;
   const float *i_bias, *f_bias;
+  // WHOLE: the norm behind, weight [H * DV], the gate's logits at g_at
+  const float* weight;
+  int g_at;
+  float eps, denom_eps;
 };
+constexpr int kMemWhole = 4;   // blocks of kMemCols columns that a workgroup of WHOLE takes at most
 
-template <int R, bool SPACE>
-__global__ __launch_bounds__(256) void memory_token_kernel(const float* __restrict__ raw, long ld, SpaceArgs sp, ExpArgs ex,
+template <int R, bool SPACE, bool WHOLE, typename T>
+__global__ __launch_bounds__(WHOLE ? 256 * kMemWhole : 256) void memory_token_kernel(const float* __restrict__ raw, long ld, SpaceArgs sp, ExpArgs ex,
                                                            int H, int N, int DV, const SeqMeta* __restrict__ seqs,
                                                            float* __restrict__ state, long state_stride, int state_vec,
-                                                           Gate* __restrict__ gates, float* __restrict__ out, long ldo) {
+                                                           Gate* __restrict__ gates, float* __restrict__ out, long ldo,
+                                                           T* __restrict__ normed, long ldn) {
   constexpr bool NORM = !SPACE;
-  __shared__ __attribute__((aligned(16))) float v_s[kMemCols];
-  __shared__ float k_s[kMemMaxRows], q_s[kMemMaxRows], part_s[4][kMemCols + 1];
-  const int blocks = (DV + kMemCols - 1) / kMemCols;
-  const int h = blockIdx.x / blocks, cb = blockIdx.x % blocks;
+  constexpr int SUBS = WHOLE ? kMemWhole : 1;
+  __shared__ __attribute__((aligned(16))) float v_all[SUBS][kMemCols];
+  __shared__ float k_s[kMemMaxRows], q_s[kMemMaxRows], part_all[SUBS][4][kMemCols + 1], o_s[SUBS * kMemCols], nq_s;
+  const int blocks = WHOLE ? 1 : (DV + kMemCols - 1) / kMemCols;
+  const int sub = WHOLE ? (int)threadIdx.x >> 8 : 0, tid = threadIdx.x & 255;
+  const int h = blockIdx.x / blocks, cb = WHOLE ? sub : blockIdx.x % blocks;
+  float* v_s = v_all[sub];
+  float(*part_s)[kMemCols + 1] = part_all[sub];
   const SeqMeta m = seqs[blockIdx.y];
   const long t = m.q_off;
   const int pos = m.q_start;
   const float* row = raw + t * ld;
-  const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
-  const int c4 = threadIdx.x & 7, group = threadIdx.x >> 3;
+  const int lane = tid & 63, w = tid >> 6;
+  const int c4 = tid & 7, group = tid >> 3;
   const int col = cb * kMemCols + 4 * c4;
   float* slot = state + (long)m.table_row * state_stride;
   float* mine = slot + (long)h * N * DV;
   float* my_n = slot + (long)H * N * DV + (long)h * N;
   MemoryColumns<R, NORM> mem;
   mem.load(mine, my_n, group, N, DV, col, state_vec != 0);   // (on its way while the operands are formed)
+  constexpr int PER = kMemWhole * kMemCols / 64;
+  float gate_v[PER], weight_v[PER];
+  if constexpr (WHOLE) {   // what the first wave applies at the end
+#pragma unroll
+    for (int j = 0; j < PER; ++j) {
+      const int c = min((int)threadIdx.x % 64 + 64 * j, DV - 1);
+      gate_v[j] = row[ex.g_at + h * DV + c];
+      weight_v[j] = ex.weight[(long)h * DV + c];
+    }
+  }
   float a, b, d = 0.f, floor = 1.0f;
   if constexpr (SPACE) {
     const int each = H / sp.G, g = h / each, inner = H * DV;
     const bool writes_group = cb == 0 && h == g * each;
     float* ring = slot + sp.ring_at;
     const int own_row = pos % sp.M, first_row = own_row + 1;   // (position pos - (M-1) + j lies in row (pos + 1 + j) mod M)
-    for (int i = threadIdx.x; i < 2 * N + kMemCols; i += 256) {
+    for (int i = tid; i < 2 * N + kMemCols; i += 256) {
       const bool is_v = i >= 2 * N;
       const int vc = cb * kMemCols + i - 2 * N;
       if (is_v && vc >= DV) {
@@ -427,7 +449,7 @@ __global__ __launch_bounds__(256) void memory_token_kernel(const float* __restri
     b = dt;
     d = sp.skip[h];
   } else {
-    for (int i = threadIdx.x; i < 2 * N + kMemCols; i += 256) {
+    for (int i = tid + (sub ? 2 * N : 0); i < 2 * N + kMemCols; i += 256) {
       if (i < N) k_s[i] = row[ex.k_at + h * N + i];
       else if (i < 2 * N) q_s[i - N] = row[ex.q_at + h * N + i - N] * ex.q_scale;
       else v_s[i - 2 * N] = cb * kMemCols + i - 2 * N < DV ? row[ex.v_at + h * DV + cb * kMemCols + i - 2 * N] : 0.f;
@@ -437,7 +459,7 @@ __global__ __launch_bounds__(256) void memory_token_kernel(const float* __restri
     float* kept = slot + ex.m_at + 4 * h;
     const double before = kept_maximum(kept + 2 * (pos & 1));
     const double now = fmax((double)gf + before, (double)gi);
-    if (cb == 0 && threadIdx.x == 0) keep_maximum(kept + 2 * ((pos + 1) & 1), now);
+    if (cb == 0 && tid == 0) keep_maximum(kept + 2 * ((pos + 1) & 1), now);
     a = expf(fminf((float)(((double)gf + before) - now), 0.f));
     b = expf((float)((double)gi - now));
     floor = expf((float)-now);
@@ -464,6 +486,27 @@ __global__ __launch_bounds__(256) void memory_token_kernel(const float* __restri
     if (NORM && lane == 0) part_s[w][kMemCols] = nq;
   }
   __syncthreads();
+  if constexpr (WHOLE) {
+    if (tid < kMemCols) o_s[cb * kMemCols + tid] = ((part_s[0][tid] + part_s[1][tid]) + part_s[2][tid]) + part_s[3][tid];
+    if (threadIdx.x == 64) nq_s = ((part_s[0][kMemCols] + part_s[1][kMemCols]) + part_s[2][kMemCols]) + part_s[3][kMemCols];
+    __syncthreads();
+    if (threadIdx.x >= 64) return;
+    const float share = 1.0f / (fmaxf(fabsf(nq_s), floor) + ex.denom_eps);
+    float v[PER], part = 0.f;   // lane i: the elements i, i + 64, ... ascending, then a butterfly
+#pragma unroll
+    for (int j = 0; j < PER; ++j) {
+      const int c = lane + 64 * j;
+      v[j] = c < DV ? o_s[c] * share : 0.f;
+      part = part + v[j] * v[j];
+    }
+    const float scale = 1.0f / sqrtf(wave_sum(part) / (float)DV + ex.eps);
+#pragma unroll
+    for (int j = 0; j < PER; ++j) {
+      const int c = lane + 64 * j;
+      if (c < DV) normed[t * ldn + (long)h * DV + c] = from_f32<T>(((v[j] * scale) * weight_v[j]) * sigmoid_m(gate_v[j]));
+    }
+    return;
+  }
   if (threadIdx.x < kMemCols) {
     const int at = threadIdx.x, c = cb * kMemCols + at;
     if (c < DV)
@@ -789,6 +832,7 @@ static int rows_vec(const float* p, long ld, int each) { return aligned16(p) && 
 
 extern "C" int ls_memory_max_rows() { return kMemMaxRows; }
 extern "C" int ls_memory_chunk() { return kChunk; }
+extern "C" int ls_exp_token_whole() { return kMemWhole * kMemCols; }
 
 extern "C" int ls_conv_gates(const float* raw, long ld, int x_at, int dt_at, int n_tokens, int C, int H, int M, const float* taps,
                              const float* bias, const float* a_log, const float* dt_bias, const int* tok_seq, const int* tok_pos,
@@ -869,8 +913,8 @@ extern "C" int ls_space_token(const float* raw, long ld, int x_at, int dt_at, in
   const int state_vec = DV % 4 == 0 && state_stride % 4 == 0 && aligned16(state);
   const dim3 grid((unsigned)(H * ((DV + kMemCols - 1) / kMemCols)), (unsigned)n_seqs);
 #define LS_TOKEN(R_)                                                                                                          \
-  hipLaunchKernelGGL((memory_token_kernel<R_, true>), grid, dim3(256), 0, s, raw, ld, sp, ex, H, N, DV, (const SeqMeta*)seqs, \
-                     state, state_stride, state_vec, (Gate*)nullptr, out, ldo);
+  hipLaunchKernelGGL((memory_token_kernel<R_, true, false, float>), grid, dim3(256), 0, s, raw, ld, sp, ex, H, N, DV,         \
+                     (const SeqMeta*)seqs, state, state_stride, state_vec, (Gate*)nullptr, out, ldo, (float*)nullptr, 0L);
   LS_BY_ROWS(LS_TOKEN)
 #undef LS_TOKEN
   return check_launch("space_token");
@@ -879,22 +923,35 @@ extern "C" int ls_space_token(const float* raw, long ld, int x_at, int dt_at, in
 extern "C" int ls_exp_token(const float* raw, long ld, int q_at, int k_at, int v_at, int i_at, int f_at, long m_at,
                             const float* i_bias, const float* f_bias, float cap, float q_scale, int H, int N, int DV,
                             const void* seqs, int n_seqs, float* state, long state_stride, float* gates, float* out, long ldo,
+                            int normed_dtype, const float* weight, int g_at, float eps, float denom_eps, void* normed, long ldn,
                             void* stream) {
+  // normed (or null): the head's norm and gate in the same launch (ls_exp_token_whole() columns at most); else gates, out
+  LS_REQUIRE(!normed || (DV <= kMemWhole * kMemCols && weight && g_at >= 0 && ld >= (long)g_at + (long)H * DV && ldn >= (long)H * DV && eps > 0.f &&
+                         (normed_dtype == kF32 || normed_dtype == kBF16)),
+             "exp_token: the norm behind takes heads of up to %d columns", kMemWhole * kMemCols);
   LS_REQUIRE(n_seqs > 0 && n_seqs <= 65535 && H > 0 && N > 0 && N <= kMemMaxRows && DV > 0 && cap > 0.f,
              "exp_token: bad sizes (%d heads, %d rows of at most %d, %d columns)", H, N, kMemMaxRows, DV);
   LS_REQUIRE(q_at >= 0 && k_at >= 0 && v_at >= 0 && i_at >= 0 && f_at >= 0 && ld >= (long)q_at + (long)H * N && ld >= (long)k_at + (long)H * N &&
                  ld >= (long)v_at + (long)H * DV && ld >= (long)i_at + H && ld >= (long)f_at + H,
              "exp_token: the projections do not fit the rows");
-  LS_REQUIRE(m_at >= (long)H * N * DV + (long)H * N && state_stride >= m_at + 4L * H && ldo >= (long)H * DV, "exp_token: state or output too short");
-  LS_REQUIRE(raw && i_bias && f_bias && seqs && state && gates && out, "exp_token: null operand");
+  LS_REQUIRE(m_at >= (long)H * N * DV + (long)H * N && state_stride >= m_at + 4L * H && (normed || ldo >= (long)H * DV), "exp_token: state or output too short");
+  LS_REQUIRE(raw && i_bias && f_bias && seqs && state && (normed || (gates && out)), "exp_token: null operand");
   hipStream_t s = reinterpret_cast<hipStream_t>(stream);
   const SpaceArgs sp{};
-  const ExpArgs ex{q_at, k_at, v_at, i_at, f_at, m_at, cap, q_scale, i_bias, f_bias};
+  const ExpArgs ex{q_at, k_at, v_at, i_at, f_at, m_at, cap, q_scale, i_bias, f_bias, weight, g_at, eps, denom_eps};
   const int state_vec = DV % 4 == 0 && state_stride % 4 == 0 && aligned16(state);
   const dim3 grid((unsigned)(H * ((DV + kMemCols - 1) / kMemCols)), (unsigned)n_seqs);
+  const dim3 whole_grid((unsigned)H, (unsigned)n_seqs), whole_block(256 * (unsigned)((DV + kMemCols - 1) / kMemCols));
 #define LS_TOKEN(R_)                                                                                                           \
-  hipLaunchKernelGGL((memory_token_kernel<R_, false>), grid, dim3(256), 0, s, raw, ld, sp, ex, H, N, DV, (const SeqMeta*)seqs, \
-                     state, state_stride, state_vec, (Gate*)gates, out, ldo);
+  if (normed && normed_dtype == kF32)                                                                                          \
+    hipLaunchKernelGGL((memory_token_kernel<R_, false, true, float>), whole_grid, whole_block, 0, s, raw, ld, sp, ex, H, N, DV, \
+                       (const SeqMeta*)seqs, state, state_stride, state_vec, (Gate*)gates, out, ldo, (float*)normed, ldn);     \
+  else if (normed)                                                                                                             \
+    hipLaunchKernelGGL((memory_token_kernel<R_, false, true, bf16_t>), whole_grid, whole_block, 0, s, raw, ld, sp, ex, H, N, DV, \
+                       (const SeqMeta*)seqs, state, state_stride, state_vec, (Gate*)gates, out, ldo, (bf16_t*)normed, ldn);    \
+  else                                                                                                                         \
+    hipLaunchKernelGGL((memory_token_kernel<R_, false, false, float>), grid, dim3(256), 0, s, raw, ld, sp, ex, H, N, DV,       \
+                       (const SeqMeta*)seqs, state, state_stride, state_vec, (Gate*)gates, out, ldo, (float*)nullptr, 0L);
   LS_BY_ROWS(LS_TOKEN)
 #undef LS_TOKEN
   return check_launch("exp_token");

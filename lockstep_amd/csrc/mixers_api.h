@@ -166,13 +166,16 @@ int ls_memory_chunks(const float* q, long ldq, int q_each, int q_share, const fl
                      int norm, const void* seqs, const int* items, int n_items, const int* runs, int n_runs, float* states, long E,
                      float* decays, float* state, long state_stride, float* out, long ldo, void* stream);
 // A step of single tokens in one launch: convolution and gates (space_token) or exponential gates (exp_token), the update
-// and the read.
+// and the read.  With `normed` (heads of at most ls_exp_token_whole() columns) exp_token also does what head_norm_gate does
+// behind it (weight [H * DV], the sigmoid of the logits at g_at) and writes neither gates nor out.
 int ls_space_token(const float* raw, long ld, int x_at, int dt_at, int C, int G, int M, long ring_at, const float* taps,
                    const float* conv_bias, const float* a_log, const float* dt_bias, const float* skip, int H, int N, int DV,
                    const void* seqs, int n_seqs, float* state, long state_stride, float* out, long ldo, void* stream);
 int ls_exp_token(const float* raw, long ld, int q_at, int k_at, int v_at, int i_at, int f_at, long m_at, const float* i_bias,
                  const float* f_bias, float cap, float q_scale, int H, int N, int DV, const void* seqs, int n_seqs, float* state,
-                 long state_stride, float* gates, float* out, long ldo, void* stream);
+                 long state_stride, float* gates, float* out, long ldo, int normed_dtype, const float* weight, int g_at, float eps,
+                 float denom_eps, void* normed, long ldn, void* stream);
+int ls_exp_token_whole();
 // y * silu(z), divided by its root mean square in each of `parts` equal runs, times weight [inner].
 int ls_gated_parts_norm(int out_dtype, const float* y, long ldy, const float* z, long ldz, int n_tokens, int inner, int parts,
                         const float* weight, float eps, void* out, long ldo, void* stream);

@@ -1171,10 +1171,49 @@ class Kernels:
             _ptr(expert), _ptr(weight), _ptr(order), _ptr(tiles), c_int(cap), _ptr(counts), c_int(("softmax", "sigmoid", "softmax_all").index(scoring)),
             _ptr(correction), c_int(count), c_int(keep), _stream()))
 
+    def experts_route_product_ok(self, dtype: torch.dtype, n_tokens: int, experts: int, top: int, k: int) -> bool:
+        """Whether ``experts_route_product`` takes a step of this many tokens of ``k`` elements."""
+        return self._memo(("route_product", dtype, n_tokens, experts, top, k), lambda: bool(self.experts_lib().ls_experts_route_product_ok(
+            c_int(DTYPE_CODE[dtype]), c_int(n_tokens), c_int(experts), c_int(top), c_int(k))))
+
+    def experts_route_product(self, x: torch.Tensor, w_router: torch.Tensor, bias, top: int, rows_a_tile: int, expert: torch.Tensor,
+                              weight: torch.Tensor, order: torch.Tensor, tiles: torch.Tensor, scoring: str = "softmax", correction=None,
+                              groups: tuple[int, int] = (1, 1)) -> None:
+        """``experts_route`` of the logits ``x @ w_router.T`` (float32 sums) for a few tokens, the product in the same launch."""
+        _rows_ok(x, "experts_route_product x")
+        if scoring not in ("softmax", "sigmoid", "softmax_all"):
+            raise KernelError(f"experts_route_product: scoring is softmax, sigmoid or softmax_all, got {scoring!r}")
+        t, k = x.shape
+        if not (w_router.is_cuda and w_router.dim() == 2 and w_router.is_contiguous() and w_router.shape[1] == k
+                and w_router.dtype == x.dtype and x.dtype in DTYPE_CODE):
+            raise KernelError("experts_route_product: the router's matrix must be [E, K] in the dtype of x")
+        e = w_router.shape[0]
+        if not (0 < top <= min(e, self.experts_max_top()) and self.experts_route_product_ok(x.dtype, t, e, top, k)):
+            raise KernelError(f"experts_route_product does not take {t} tokens, {top} of {e} experts")
+        count, keep = groups
+        if bias is not None:
+            self._f32_vector(bias, e, "experts_route_product bias")
+        if scoring == "softmax_all":
+            self._f32_vector(correction, e, "experts_route_product correction")
+            if not (0 < keep <= count and e % count == 0 and top <= keep * (e // count)):
+                raise KernelError(f"experts_route_product: {e} experts in {count} groups of which {keep} are kept, {top} a token")
+        cap = self.experts_tile_capacity(t, e, top, rows_a_tile)
+        self._i32(expert, t * top, "experts_route_product expert"); self._i32(order, t * top, "experts_route_product order")
+        self._i32(tiles, 4 * cap, "experts_route_product tiles")
+        if not (weight.is_cuda and weight.dtype == torch.float32 and weight.is_contiguous() and weight.numel() >= t * top):
+            raise KernelError("experts_route_product weight must be float32 [T, top]")
+        if t == 0:
+            return
+        lib = self.experts_lib()
+        self._launch(lib, lib.ls_experts_route_product, (
+            c_int(DTYPE_CODE[x.dtype]), _ptr(x), c_long(x.stride(0)), _ptr(w_router), c_int(k), _ptr(bias), c_int(t), c_int(e), c_int(top),
+            c_int(rows_a_tile), _ptr(expert), _ptr(weight), _ptr(order), _ptr(tiles), c_int(cap),
+            c_int(("softmax", "sigmoid", "softmax_all").index(scoring)), _ptr(correction), c_int(count), c_int(keep), _stream()))
+
     def experts_apply(self, x: torch.Tensor, w_gate: torch.Tensor, w_up: torch.Tensor, w_down: torch.Tensor, top: int,
                       rows_a_tile: int, order: torch.Tensor, tiles: torch.Tensor, weight: torch.Tensor, limit: float,
                       alpha: float, act: torch.Tensor, partials: torch.Tensor, shift: float = 1.0,
-                      weigh_input: bool = False, identity: int = 0) -> None:
+                      weigh_input: bool = False, identity: int = 0, shared=None) -> None:
         """``partials[k][t] = weight[t, k] * down_e(act(gate_e x[t], up_e x[t]))`` for every token's ``k``-th
         expert ``e``, with the clamped gated unit of ``glu_clamped`` as activation (``min(g, limit) sigmoid(alpha
         min(g, limit)) (clamp(u, -limit, limit) + shift)``; an infinite ``limit``, ``alpha`` 1 and ``shift`` 0 are the
@@ -1182,7 +1221,10 @@ class Kernels:
         ``[E, F, K]``, ``w_down [E, N, F]`` in the compute dtype; ``act``: scratch ``[T * top, F]`` of the
         compute dtype; ``partials [top, T, N]`` float32; the routing as ``experts_route`` left it.
         ``weigh_input``: the weight multiplies the expert's input instead, ``partials[k][t] = down_e(act(w gate_e
-        x[t], w up_e x[t]))``.  ``identity``: that many experts behind those with weights return their input."""
+        x[t], w up_e x[t]))``.  ``identity``: that many experts behind those with weights return their input.
+        ``shared`` (tiles of 16 rows only): an expert that every token uses, worked on in the same launches, as (its gate and
+        up rows interleaved in tiles of 16, its down matrix ``[N, Fs]``, scratch ``[T, Fs]`` of the compute dtype, float32
+        ``[T, N]`` for its output)."""
         _rows_ok(x, "experts_apply x"); _rows_ok(act, "experts_apply act")
         t, k = x.shape
         if not (w_gate.dim() == 3 and w_gate.shape == w_up.shape and w_gate.shape[2] == k and w_down.dim() == 3
@@ -1203,6 +1245,18 @@ class Kernels:
         self._i32(order, t * top, "experts_apply order"); self._i32(tiles, 4 * cap, "experts_apply tiles")
         if not (weight.is_cuda and weight.dtype == torch.float32 and weight.is_contiguous() and weight.numel() >= t * top):
             raise KernelError("experts_apply weight must be float32 [T, top]")
+        gate_up = down = sh_act = sh_out = None
+        sh_f = sh_ld = 0
+        if shared is not None:
+            gate_up, down, sh_act, sh_out = shared
+            sh_f = down.shape[1]
+            _rows_ok(sh_act, "experts_apply shared act"); _rows_ok(sh_out, "experts_apply shared out")
+            if not (rows_a_tile == 16 and gate_up.is_cuda and gate_up.is_contiguous() and down.is_contiguous() and gate_up.dtype == down.dtype
+                    == sh_act.dtype == x.dtype and tuple(gate_up.shape) == (-(-sh_f // 16) * 32, k) and down.shape[0] == n
+                    and sh_act.shape[0] >= t and sh_act.shape[1] == sh_f and sh_out.dtype == torch.float32 and sh_out.is_contiguous()
+                    and tuple(sh_out.shape) == (t, n)):
+                raise KernelError("experts_apply: the shared expert's operands do not fit, or the tiles have more than 16 rows")
+            sh_ld = sh_act.stride(0)
         if t == 0:
             return
         lib = self.experts_lib()
@@ -1210,7 +1264,8 @@ class Kernels:
             c_int(DTYPE_CODE[x.dtype]), _ptr(x), c_long(x.stride(0)), _ptr(w_gate), _ptr(w_up), _ptr(w_down), c_int(t),
             c_int(e), c_int(top), c_int(k), c_int(f), c_int(n), c_int(rows_a_tile), _ptr(order), _ptr(tiles), c_int(cap),
             _ptr(weight), c_float(limit), c_float(alpha), c_float(shift), _ptr(act), c_long(act.stride(0)), _ptr(partials),
-            c_int(int(bool(weigh_input))), c_int(real), _stream()))
+            c_int(int(bool(weigh_input))), c_int(real), _ptr(gate_up), _ptr(down), c_int(sh_f), _ptr(sh_act), c_long(sh_ld),
+            _ptr(sh_out), _stream()))
 
     def experts_route_table(self, token_ids: torch.Tensor, table: torch.Tensor, experts: int, rows_a_tile: int,
                             expert: torch.Tensor, weight: torch.Tensor, order: torch.Tensor, tiles: torch.Tensor,
@@ -1778,25 +1833,39 @@ class Kernels:
 
     def exp_token(self, raw: torch.Tensor, q_at: int, k_at: int, v_at: int, i_at: int, f_at: int, i_bias, f_bias, cap: float,
                   q_scale: float, heads: int, rows: int, vdim: int, seqs, n_seqs: int, state: torch.Tensor, max_at: int,
-                  gates: torch.Tensor, out: torch.Tensor) -> None:
-        """A step of single tokens of a memory with exponential gates in one launch: what ``exp_gates`` and ``memory`` do."""
+                  gates, out: torch.Tensor, normed=None) -> None:
+        """A step of single tokens of a memory with exponential gates in one launch: what ``exp_gates`` and ``memory`` do.
+        ``normed`` (heads of at most ``exp_token_whole()`` columns): (weight ``[heads*vdim]``, column of the gate's logits, eps,
+        denom_eps); ``out`` then gets what ``head_norm_gate`` would leave, in its dtype, and there are no ``gates``."""
         _rows_ok(raw, "exp_token raw"); _rows_ok(out, "exp_token out")
         if not (raw.dtype == torch.float32 and cap > 0 and min(q_at, k_at, v_at, i_at, f_at) >= 0 and raw.shape[0] >= n_seqs
                 and raw.shape[1] >= max(max(q_at, k_at) + heads * rows, v_at + heads * vdim, max(i_at, f_at) + heads)):
             raise KernelError("exp_token: the projections do not fit the float32 rows, or the cap is not positive")
         self._f32_vector(i_bias, heads, "exp_token i_bias"); self._f32_vector(f_bias, heads, "exp_token f_bias")
         self._memory_state(state, max_at + 4 * heads, "exp_token")
-        self._gates_ok(gates, n_seqs, heads, "exp_token")
         self._seqs_ok(seqs, n_seqs, "exp_token")
-        if not (out.dtype == torch.float32 and tuple(out.shape) == (n_seqs, heads * vdim)):
-            raise KernelError(f"exp_token out must be float32 [{n_seqs}, {heads * vdim}]")
+        weight, g_at, eps, denom_eps = normed if normed is not None else (None, 0, 0.0, 0.0)
+        if normed is None:
+            self._gates_ok(gates, n_seqs, heads, "exp_token")
+        else:
+            self._f32_vector(weight, heads * vdim, "exp_token weight")
+            if not (vdim <= self.exp_token_whole() and 0 <= g_at <= raw.shape[1] - heads * vdim and eps > 0):
+                raise KernelError(f"exp_token: the norm behind takes heads of up to {self.exp_token_whole()} columns and a gate inside the rows")
+        if not (out.dtype in DTYPE_CODE and (normed is not None or out.dtype == torch.float32) and tuple(out.shape) == (n_seqs, heads * vdim)):
+            raise KernelError(f"exp_token out must be [{n_seqs}, {heads * vdim}], float32 without a norm behind")
         if n_seqs == 0:
             return
         lib = self.mixers_lib()
         self._launch(lib, lib.ls_exp_token, (
             _ptr(raw), c_long(raw.stride(0)), c_int(q_at), c_int(k_at), c_int(v_at), c_int(i_at), c_int(f_at), c_long(max_at),
             _ptr(i_bias), _ptr(f_bias), c_float(cap), c_float(q_scale), c_int(heads), c_int(rows), c_int(vdim), _ptr(seqs),
-            c_int(n_seqs), _ptr(state), c_long(state.stride(0)), _ptr(gates), _ptr(out), c_long(out.stride(0)), _stream()))
+            c_int(n_seqs), _ptr(state), c_long(state.stride(0)), _ptr(gates if normed is None else None),
+            _ptr(out if normed is None else None), c_long(out.stride(0)), c_int(DTYPE_CODE[out.dtype]), _ptr(weight), c_int(g_at),
+            c_float(eps), c_float(denom_eps), _ptr(out if normed is not None else None), c_long(out.stride(0)), _stream()))
+
+    def exp_token_whole(self) -> int:
+        """Columns a head may have for ``exp_token`` to norm it in the same launch."""
+        return self._memo(("exp_token_whole",), lambda: int(self.mixers_lib().ls_exp_token_whole()))
 
     def gated_parts_norm(self, y: torch.Tensor, z: torch.Tensor, parts: int, weight, eps: float, out: torch.Tensor) -> None:
         """``y * silu(z)``, divided by its root mean square in each of ``parts`` equal runs of a row (``eps`` inside the

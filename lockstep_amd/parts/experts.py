@@ -162,6 +162,9 @@ class RoutedExperts(FeedForward):
         counts = ctx.buf("experts.counts", (e,), torch.int32)
         if self.tabled:
             k.experts_route_table(ctx.token_ids, self.table, e, rows, chosen, share, order, tiles, counts)
+        elif k.experts_route_product_ok(rt.dtype, t, e, top, self.hidden):          # a few tokens: the router's product in the same launch
+            k.experts_route_product(x, self.w_router, self.b_router, top, rows, chosen, share, order, tiles, scoring=self.score,
+                                    correction=self.correction, groups=self.groups)
         else:
             logits = ctx.buf("experts.logits", (t, e), torch.float32)
             k.gemm(x, self.w_router, logits, STORE_F32)
@@ -170,9 +173,14 @@ class RoutedExperts(FeedForward):
         slices = top + (1 if self.shared is not None else 0)
         partials = ctx.buf("experts.slices", (slices * t, self.hidden), torch.float32).view(slices, t, self.hidden)
         act = ctx.buf("experts.act", (t * top, self.inter), rt.dtype)
+        # few tokens an expert: a shared expert with the plain gated unit is worked on in the experts' own launches
+        beside = None
+        if rows == 16 and self.shared is not None and getattr(self.shared, "kind", "") == "gated_mlp" and self.shared.fused:
+            beside = (self.shared.w_gate_up, self.shared.w_down, ctx.buf("experts.shared_act", (t, self.shared.inter), rt.dtype),
+                      partials[top])
         k.experts_apply(x, self.w_gate, self.w_up, self.w_down, top, rows, order, tiles, share, self.limit, self.alpha,
-                        act, partials[:top], shift=self.shift, weigh_input=self.weigh == "input", identity=self.identity)
-        if self.shared is not None:
+                        act, partials[:top], shift=self.shift, weigh_input=self.weigh == "input", identity=self.identity, shared=beside)
+        if self.shared is not None and beside is None:
             self.shared.forward(ctx, x, partials[top], accumulate=False)
         pending = PendingAdd(partials)
         if defer == "any" or (defer and t <= DEFER_ROWS and self.hidden % 4 == 0):

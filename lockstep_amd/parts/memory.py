@@ -238,9 +238,13 @@ class MatrixMemory(_Memory):
         g_at, i_at = v_at + n * dv, v_at + 2 * n * dv
         f_at = i_at + n
         state = ctx.cache.unit_state(run.cache)
+        scale = d ** -0.5
+        if ctx.single_tokens and dv <= k.exp_token_whole():           # the head's norm and gate in the same launch
+            k.exp_token(raw, 0, k_at, v_at, i_at, f_at, self.i_bias, self.f_bias, self.cap, scale, n, d, dv, ctx.seqs, ctx.n_seqs, state,
+                        self.max_at, None, out, normed=(self.norm_weight, g_at, self.eps, self.denom_eps))
+            return
         o = ctx.buf("memory.y", (t, n * dv), torch.float32)
         gates = ctx.buf("memory.gates", (t * n * k.GATE_FLOATS,), torch.float32)
-        scale = d ** -0.5
         if ctx.single_tokens:
             k.exp_token(raw, 0, k_at, v_at, i_at, f_at, self.i_bias, self.f_bias, self.cap, scale, n, d, dv, ctx.seqs, ctx.n_seqs, state,
                         self.max_at, gates, o)

@@ -262,7 +262,7 @@ def test_the_state_space_mixer_over_unequal_requests_in_steps(dtype, heads, grou
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
 @pytest.mark.parametrize("heads, rows, dv, cap", [(3, 20, 24, 8.0), (1, 1, 5, 3.0), (2, 70, 9, 20.0), (4, 128, 128, 15.0), (2, 256, 40, 2.0),
-                                                  (5, 33, 66, 10.0)])
+                                                  (5, 33, 66, 10.0), (2, 48, 150, 6.0)])
 def test_the_matrix_memory_over_unequal_requests_in_steps(dtype, heads, rows, dv, cap):
     g = torch.Generator().manual_seed(heads * rows + dv)
     draw = lambda *s: torch.randn(s, generator=g)  # noqa: E731
@@ -319,6 +319,68 @@ def test_the_choice_of_experts_in_groups(tokens, routed, top, groups, keep):
     placed = order.cpu().long()
     assert sorted(placed.tolist()) == list(range(tokens * top))
     assert bool((expert.cpu()[placed].diff() >= 0).all())
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("tokens, routed, top, kk, scoring", [(1, 8, 2, 64, "softmax_all"), (16, 36, 4, 1000, "softmax_all"), (7, 128, 6, 136, "softmax_all"),
+                                                              (13, 18, 3, 40, "softmax"), (3, 100, 5, 512, "sigmoid"), (2, 1, 1, 24, "softmax")])
+def test_the_routers_product_in_the_routing_launch(dtype, tokens, routed, top, kk, scoring):
+    """Logits that are small whole numbers (exact in any order of sums): the same choices and weights as from given logits."""
+    g = torch.Generator().manual_seed(routed + tokens)
+    x = torch.randint(-2, 3, (tokens, kk + 7), generator=g).to(dtype)
+    w = (torch.randint(-1, 2, (routed, kk), generator=g) * (torch.rand((routed, kk), generator=g) < 0.1)).to(dtype)
+    bias = torch.randn(routed, generator=g) * 0.01                       # (no ties)
+    correction = torch.randn(routed, generator=g) if scoring == "softmax_all" else None
+    logits = x[:, :kk].float() @ w.float().T
+    k = K()
+    cap = k.experts_tile_capacity(tokens, routed, top, 16)
+    got = []
+    for product in (True, False):
+        expert, order = (torch.full((tokens * top,), -7, dtype=torch.int32, device="cuda") for _ in range(2))
+        share, tiles = torch.empty(tokens * top, device="cuda"), torch.full((4 * cap,), -7, dtype=torch.int32, device="cuda")
+        more = dict(scoring=scoring, correction=None if correction is None else correction.cuda())
+        if product:
+            assert k.experts_route_product_ok(dtype, tokens, routed, top, kk)
+            # (rows of a wider buffer, on 16-byte boundaries)
+            wide = torch.full((tokens, -(-kk // 8) * 8 + 8), float("nan"), dtype=dtype, device="cuda")
+            wide[:, :kk] = x[:, :kk].cuda()
+            k.experts_route_product(wide[:, :kk], w.cuda(), bias.cuda(), top, 16, expert, share, order, tiles, **more)
+        else:
+            counts = torch.empty(routed, dtype=torch.int32, device="cuda")
+            k.experts_route(logits.cuda(), bias.cuda(), top, 16, expert, share, order, tiles, counts, **more)
+        got.append((expert.cpu(), order.cpu(), tiles.cpu(), share.cpu()))
+    for a, b in zip(*got):
+        assert torch.equal(a, b)
+    assert not k.experts_route_product_ok(dtype, 17, routed, top, kk) and not k.experts_route_product_ok(dtype, tokens, routed, top, kk + 1)
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("tokens, experts, top, width, ff, shared_ff", [(1, 4, 2, 64, 32, 96), (33, 9, 2, 96, 48, 20), (5, 3, 1, 45, 9, 33), (16, 8, 4, 128, 16, 16)])
+def test_a_shared_expert_in_the_routed_experts_launches(dtype, tokens, experts, top, width, ff, shared_ff):
+    from lockstep_amd.ops import interleave_gate_up
+
+    g = torch.Generator().manual_seed(tokens + width)
+    draw = lambda *s: (torch.randn(s, generator=g) * 0.3).to(dtype)  # noqa: E731
+    x = (torch.randn((tokens, width), generator=g)).to(dtype)
+    w_gate, w_up, w_down = draw(experts, ff, width), draw(experts, ff, width), draw(experts, width, ff)
+    s_gate, s_up, s_down = draw(shared_ff, width), draw(shared_ff, width), draw(width, shared_ff)
+    logits = torch.randn((tokens, experts), generator=g)
+    k = K()
+    cap = k.experts_tile_capacity(tokens, experts, top, 16)
+    expert, order = (torch.empty(tokens * top, dtype=torch.int32, device="cuda") for _ in range(2))
+    share, tiles = torch.empty(tokens * top, device="cuda"), torch.empty(4 * cap, dtype=torch.int32, device="cuda")
+    k.experts_route(logits.cuda(), None, top, 16, expert, share, order, tiles, torch.empty(experts, dtype=torch.int32, device="cuda"))
+    act = torch.empty((tokens * top, ff), dtype=dtype, device="cuda")
+    args = (x.cuda(), w_gate.cuda(), w_up.cuda(), w_down.cuda(), top, 16, order, tiles, share, float("inf"), 1.0, act)
+    alone, beside = (torch.full((top + 1, tokens, width), float("nan"), device="cuda") for _ in range(2))
+    k.experts_apply(*args, alone[:top], shift=0.0)
+    sh_act = torch.empty((tokens, shared_ff), dtype=dtype, device="cuda")
+    k.experts_apply(*args, beside[:top], shift=0.0,
+                    shared=(interleave_gate_up(s_gate, s_up).cuda(), s_down.cuda(), sh_act, beside[top]))
+    assert torch.equal(alone[:top], beside[:top])
+    xd = x.double()
+    want = (plain.silu(xd @ s_gate.double().T) * (xd @ s_up.double().T)) @ s_down.double().T
+    assert close(beside[top], want, dtype, scale=0.1), float((beside[top].double().cpu() - want).abs().max())
 
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
